@@ -13,7 +13,7 @@ from dataclasses import dataclass
 from typing import Callable, Dict
 
 from .specs import (AttentionSpec, BandScaledRopeSpec, ParallelMixerSpec, SSDSpec, ConfigError, DecayAttentionSpec, EmbeddingSpec, GatedDeltaSpec, GatedMLPSpec,
-                    HeadSpec, HyperConnectionSpec, LatentAttentionSpec, LayerNormSpec, LayerRun, LayerSpec, MLSTMSpec,
+                    GatedRecurrenceSpec, HeadSpec, HyperConnectionSpec, LatentAttentionSpec, LayerNormSpec, LayerRun, LayerScaleSpec, LayerSpec, MLSTMSpec,
                     MixedHeadAttentionSpec, ModelSpec, NoPositionSpec, OnePlusRMSNormSpec, RMSNormSpec, RopeSpec,
                     RoutedMLPSpec, ScaledRopeSpec)
 
@@ -114,3 +114,8 @@ from . import zivazen as _zivazen  # noqa: E402
 
 register_architecture(_zivazen.ARCHITECTURE, _zivazen.ZivazenConfig.from_dict)
 ZivazenConfig = _zivazen.ZivazenConfig
+
+from . import bipazen as _bipazen  # noqa: E402
+
+register_architecture(_bipazen.ARCHITECTURE, _bipazen.BipazenConfig.from_dict)
+BipazenConfig = _bipazen.BipazenConfig

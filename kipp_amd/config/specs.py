@@ -54,6 +54,16 @@ class LayerNormSpec:
 
 
 @dataclass(frozen=True)
+class LayerScaleSpec:
+    """A factor a column on a sublayer's result: scale[c] * delta[r, c], in float32.  `name`: the tensor's local name (file
+    name = prefix + name)."""
+    width: int
+    prefix: str = ""
+    name: str = "weight"
+    kind: str = "layer_scale"
+
+
+@dataclass(frozen=True)
 class RopeSpec:
     """Rotary position encoding over the first `rotary_dim` dims of a head.
 
@@ -262,20 +272,22 @@ class LatentAttentionSpec:
     cq = N(W_dq x), q = W_uq cq, a head being [head_dim unrotated | rot_dim rotated];  W_dkv x = [c' | kr], c = N(c');
     head h: key [W_uk_h c | rot(kr)], value W_uv_h c (`v_head_dim` numbers); score = scale * q_h . key_h; position i
     sees j when 0 <= i - j < `window` (None: every j <= i); with `output_gate` head h's result is multiplied by
-    sigmoid(W_g x)_h.  N is an RMS norm with a plain weight and `norm_eps`.  `position` rotates the first
-    rotary_dim numbers of the rotated parts.  `names`: local tensor names of (dq, dq norm, uq, dkv, dkv norm, uk, uv, g, o)."""
+    sigmoid(W_g x)_h, or, `gate_each`, every number of the heads side by side by its own sigmoid(W_g x).  N is an RMS norm
+    with a plain weight and `norm_eps`.  `position` rotates the first rotary_dim numbers of the rotated parts.  `q_rank` None:
+    there is no query latent, q = W_uq x.  `names`: local tensor names of (dq, dq norm, uq, dkv, dkv norm, uk, uv, g, o)."""
     hidden_size: int
     num_heads: int
     head_dim: int
     rot_dim: int
     v_head_dim: int
-    q_rank: int
+    q_rank: Optional[int]
     kv_rank: int
     scale: float
     norm_eps: float
     position: object = NoPositionSpec()
     window: Optional[int] = None
     output_gate: bool = True
+    gate_each: bool = False
     prefix: str = ""
     kind: str = "latent_attention"
     page_size: Optional[int] = None
@@ -284,7 +296,7 @@ class LatentAttentionSpec:
     def __post_init__(self):
         for what, v in (("heads", self.num_heads), ("head_dim", self.head_dim), ("v_head_dim", self.v_head_dim),
                         ("q_rank", self.q_rank), ("kv_rank", self.kv_rank)):
-            if v <= 0:
+            if v is not None and v <= 0:
                 raise ConfigError(f"latent attention: {what} must be positive, got {v}")
         if self.rot_dim < 0:
             raise ConfigError(f"latent attention: rot_dim must not be negative, got {self.rot_dim}")
@@ -447,6 +459,36 @@ class SSDSpec:
 
 
 @dataclass(frozen=True)
+class GatedRecurrenceSpec:
+    """A recurrent block with a real-gated linear recurrent unit (Griffin): per channel a state S that starts at zero and is
+    carried from token to token in float32, beside the last inputs of a short convolution.
+
+    y = gelu_tanh(W_y x + b_y);  u = filter(W_x x + b_x) + bias, a causal filter a channel over the last `conv_taps` inputs
+    (zeros before the start, the last tap is the current token's).  u in `blocks` equal parts, in each r = sigmoid(R u + b_r) and
+    i = sigmoid(I u + b_i) with square matrices [out, in];  log a = -`factor` r softplus(lam);
+    S_t = a S_(t-1) + sqrt(1 - a^2) i u, also at the first token;  W_o (S * y).
+    `names`: local tensor names of (y, y bias, x, x bias, conv, conv bias, R, R bias, I, I bias, lam, o)."""
+    hidden_size: int
+    width: int
+    blocks: int
+    conv_taps: int
+    factor: float = 8.0
+    prefix: str = ""
+    kind: str = "gated_recurrence"
+    names: Tuple[str, ...] = ("y", "y.b", "x", "x.b", "conv", "conv.b", "ra", "ra.b", "ri", "ri.b", "lam", "o")
+
+    def __post_init__(self):
+        if self.width <= 0 or self.blocks <= 0 or self.width % self.blocks:
+            raise ConfigError(f"gated recurrence: width {self.width} must be a positive multiple of blocks {self.blocks}")
+        if not 1 <= self.conv_taps <= 16:
+            raise ConfigError(f"gated recurrence: the short convolution takes 1 to 16 taps, got {self.conv_taps}")
+        if not self.factor > 0:
+            raise ConfigError(f"gated recurrence: factor must be positive, got {self.factor}")
+        if len(self.names) != 12:
+            raise ConfigError("names: twelve local tensor names")
+
+
+@dataclass(frozen=True)
 class ParallelMixerSpec:
     """Two mixers side by side that read the same input: delta = left_scale * left(x) + right_scale * right(x).  At most one
     of them keeps keys and values in pages and at most one keeps state of fixed size."""
@@ -567,7 +609,9 @@ class RoutedMLPSpec:
     `activation` "relu2" is the square of relu.  `router` "sigmoid": scores s = sigmoid(W_router x); the choice goes by
     s + the tensor `correction_name` (None: no correction); with `groups` (count, keep) the experts form `count` equal groups
     of neighbours, a group's score is the sum of its two largest choice scores, and only experts of the `keep` best groups can
-    be chosen; weights are s / (sum of the chosen s + `weight_eps`) * `route_scale`."""
+    be chosen; weights are s / (sum of the chosen s + `weight_eps`) * `route_scale`, or, `renormalize` False, s * `route_scale`.
+    `gate_name`: an expert has a third matrix of that local name and is W_down_e (act(W_gate_e x) * (W_up_e x)) (the shared one
+    likewise).  `weigh_input`: a weight multiplies its expert's input, not its result: sum of E_e(weight_e x)."""
     hidden_size: int
     experts: int
     top: int
@@ -585,12 +629,17 @@ class RoutedMLPSpec:
     correction_name: Optional[str] = None
     groups: Optional[Tuple[int, int]] = None
     route_scale: float = 1.0
+    renormalize: bool = True
+    gate_name: Optional[str] = None
+    weigh_input: bool = False
 
     def __post_init__(self):
+        if self.weigh_input and self.gate_name is None:
+            raise ConfigError("routed feed-forward: weights on the input are implemented for experts with a gate")
         if self.router not in ("softmax", "sigmoid"):
             raise ConfigError(f"routed feed-forward: router {self.router!r} is not one of softmax, sigmoid")
-        if self.router == "softmax" and (self.correction_name is not None or self.groups is not None or self.route_scale != 1.0):
-            raise ConfigError("routed feed-forward: a correction, groups and a scale belong to the sigmoid router")
+        if self.router == "softmax" and (self.correction_name is not None or self.groups is not None or self.route_scale != 1.0 or not self.renormalize):
+            raise ConfigError("routed feed-forward: a correction, groups, a scale and weights as they are belong to the sigmoid router")
         if self.groups is not None:
             count, keep = self.groups
             if count <= 0 or self.experts % count or not 0 < keep <= count or self.top > keep * (self.experts // count):
@@ -621,6 +670,8 @@ class LayerSpec:
     x += a mixer_post_norm(mixer(mixer_norm(x))); x += a ffn_post_norm(ffn(ffn_norm(x))), a = `residual_scale`;
     "sandwich_norm_mixer" is its first half alone.  "parallel" has the roles mixer_norm, mixer and ffn: one norm whose
     output both sublayers read, h = mixer_norm(x); x += mixer(h) + ffn(h); "parallel_mixer" is the same without a feed-forward.
+    "scaled_pre_norm" is pre-norm with a scale on each sublayer's result (roles mixer_scale, ffn_scale besides):
+    x += mixer_scale(mixer(mixer_norm(x))); x += ffn_scale(ffn(ffn_norm(x))); "scaled_pre_norm_mixer" is its first half alone.
     """
     parts: Tuple[Tuple[str, object], ...]
     block: str = "pre_norm"

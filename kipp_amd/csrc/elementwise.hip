@@ -18,9 +18,10 @@ __global__ void embed_kernel(const TW* __restrict__ table, const int32_t* __rest
 // `parts` slabs [parts, rows, width] that are added in order (a product whose
 // contraction was split over workgroups), then
 // y = x * rsqrt(mean(x^2) + eps) * w   (/root/reference/src/kipp.c:2221-2231:
-// eps inside the root, (x * scale) * w).
-template <typename TD, typename TO>
-__global__ void rmsnorm_kernel(float* __restrict__ x, const TD* __restrict__ delta,
+// eps inside the root, (x * scale) * w).  With SCALED column i of the delta (its slabs
+// added first) is multiplied by dscale[i] on its way into the sum.
+template <typename TD, typename TO, bool SCALED>
+__global__ void rmsnorm_kernel(float* __restrict__ x, const TD* __restrict__ delta, const float* __restrict__ dscale,
                                const float* __restrict__ weight, TO* __restrict__ out,
                                int width, float eps, int parts, size_t part_stride) {
     __shared__ float scratch[16];
@@ -29,7 +30,13 @@ __global__ void rmsnorm_kernel(float* __restrict__ x, const TD* __restrict__ del
     for (int i = threadIdx.x; i < width; i += blockDim.x) {
         float v = x[base + i];
         if (delta != nullptr) {
-            for (int p = 0; p < parts; ++p) v += load_f(delta, p * part_stride + base + i);
+            if (SCALED) {
+                float d = 0.0f;
+                for (int p = 0; p < parts; ++p) d += load_f(delta, p * part_stride + base + i);
+                v = fmaf(dscale[i], d, v);
+            } else {
+                for (int p = 0; p < parts; ++p) v += load_f(delta, p * part_stride + base + i);
+            }
             x[base + i] = v;
         }
         ss += v * v;
@@ -57,14 +64,15 @@ __device__ __forceinline__ void store4(bf16_t* p, size_t i4, float4 v) {
     ((uint2*)p)[i4] = r;
 }
 
-template <typename TD, typename TO, int CH, int THREADS = 256>
+template <typename TD, typename TO, bool SCALED, int CH, int THREADS = 256>
 __global__ void __launch_bounds__(THREADS) rmsnorm_rows_kernel(float* __restrict__ x, const TD* __restrict__ delta,
+                                                           const float* __restrict__ dscale,
                                                            const float* __restrict__ weight, TO* __restrict__ out,
                                                            int width, float eps, int parts, size_t part_stride) {
     __shared__ float scratch[16];
     const int n4 = width / 4;
     const size_t base4 = (size_t)blockIdx.x * n4;
-    float4 v[CH], w[CH];
+    float4 v[CH], w[CH], sum[SCALED ? CH : 1], by[SCALED ? CH : 1];
     float ss = 0.0f;
     // every load is issued before anything is added: the kernel is a few round trips to memory long
 #pragma unroll
@@ -72,9 +80,11 @@ __global__ void __launch_bounds__(THREADS) rmsnorm_rows_kernel(float* __restrict
         const int i = threadIdx.x + c * THREADS;
         v[c] = make_float4(0.0f, 0.0f, 0.0f, 0.0f);
         w[c] = v[c];
+        if (SCALED) sum[c] = by[c] = v[c];
         if (i < n4) {
             v[c] = load4(x, base4 + i);
             w[c] = load4(weight, (size_t)i);
+            if (SCALED) by[c] = load4(dscale, (size_t)i);
         }
     }
     if (delta != nullptr) {
@@ -93,15 +103,22 @@ __global__ void __launch_bounds__(THREADS) rmsnorm_rows_kernel(float* __restrict
             for (int c = 0; c < CH; ++c)
 #pragma unroll
                 for (int q = 0; q < 4; ++q) {   // slabs in order
-                    v[c].x += d[c][q].x;
-                    v[c].y += d[c][q].y;
-                    v[c].z += d[c][q].z;
-                    v[c].w += d[c][q].w;
+                    float4& to = SCALED ? sum[c] : v[c];
+                    to.x += d[c][q].x;
+                    to.y += d[c][q].y;
+                    to.z += d[c][q].z;
+                    to.w += d[c][q].w;
                 }
         }
 #pragma unroll
         for (int c = 0; c < CH; ++c) {
             const int i = threadIdx.x + c * THREADS;
+            if (SCALED) {
+                v[c].x = fmaf(by[c].x, sum[c].x, v[c].x);
+                v[c].y = fmaf(by[c].y, sum[c].y, v[c].y);
+                v[c].z = fmaf(by[c].z, sum[c].z, v[c].z);
+                v[c].w = fmaf(by[c].w, sum[c].w, v[c].w);
+            }
             if (i < n4) store4(x, base4 + i, v[c]);
         }
     }
@@ -388,9 +405,9 @@ __global__ void __launch_bounds__(256) scaled_add_rmsnorm_rows_kernel(float* __r
     }
 }
 
-template <typename TD, typename TO>
+template <typename TD, typename TO, bool SCALED = false>
 static void launch_rmsnorm(float* x, const void* delta, const float* weight, void* out, int rows, int width, float eps,
-                           int parts, hipStream_t stream) {
+                           int parts, hipStream_t stream, const float* dscale = nullptr) {
     const size_t stride = (size_t)rows * width;
     const int n4 = width / 4;
     // Few rows are few workgroups, each a few round trips to memory long: a workgroup of up to 1,024 threads then takes its
@@ -399,21 +416,21 @@ static void launch_rmsnorm(float* x, const void* delta, const float* weight, voi
     // promises a row the same bits in every batch.
     constexpr bool rounds = sizeof(TO) == 2;
     if (rounds && (width & 3) == 0 && rows <= 256 && n4 > 256 && n4 <= 2048) {
-#define KIPP_RW(CH, THREADS) hipLaunchKernelGGL((rmsnorm_rows_kernel<TD, TO, CH, THREADS>), dim3(rows), dim3(THREADS), 0, stream, x, (const TD*)delta, weight, (TO*)out, width, eps, parts, stride)
+#define KIPP_RW(CH, THREADS) hipLaunchKernelGGL((rmsnorm_rows_kernel<TD, TO, SCALED, CH, THREADS>), dim3(rows), dim3(THREADS), 0, stream, x, (const TD*)delta, dscale, weight, (TO*)out, width, eps, parts, stride)
         if (n4 <= 512) KIPP_RW(1, 512);
         else if (n4 <= 1024) KIPP_RW(1, 1024);
         else KIPP_RW(2, 1024);
 #undef KIPP_RW
     } else if ((width & 3) == 0 && n4 <= 256 * 8) {
-#define KIPP_RV(CH) hipLaunchKernelGGL((rmsnorm_rows_kernel<TD, TO, CH>), dim3(rows), dim3(256), 0, stream, x, (const TD*)delta, weight, (TO*)out, width, eps, parts, stride)
+#define KIPP_RV(CH) hipLaunchKernelGGL((rmsnorm_rows_kernel<TD, TO, SCALED, CH>), dim3(rows), dim3(256), 0, stream, x, (const TD*)delta, dscale, weight, (TO*)out, width, eps, parts, stride)
         if (n4 <= 256) KIPP_RV(1);
         else if (n4 <= 512) KIPP_RV(2);
         else if (n4 <= 1024) KIPP_RV(4);
         else KIPP_RV(8);
 #undef KIPP_RV
     } else {
-        hipLaunchKernelGGL((rmsnorm_kernel<TD, TO>), dim3(rows), dim3(width >= 2048 ? 512 : 256), 0, stream, x,
-                           (const TD*)delta, weight, (TO*)out, width, eps, parts, stride);
+        hipLaunchKernelGGL((rmsnorm_kernel<TD, TO, SCALED>), dim3(rows), dim3(width >= 2048 ? 512 : 256), 0, stream, x,
+                           (const TD*)delta, dscale, weight, (TO*)out, width, eps, parts, stride);
     }
 }
 
@@ -432,6 +449,17 @@ __global__ void residual_add_scaled_kernel(float* __restrict__ x, const float* _
         for (int p = 1; p < parts; ++p) d += delta[p * n + i];
         if (bias != nullptr) d += bias[i % width];
         x[i] = fmaf(scale, d, x[i]);
+    }
+}
+
+// out[r][c] = scale[c] * (sum of the slabs of delta[r][c]), or x[r][c] += that where `add`.
+__global__ void scale_columns_kernel(float* __restrict__ x, const float* __restrict__ delta, size_t n, int parts,
+                                     const float* __restrict__ scale, int width, int add) {
+    const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+    if (i < n) {
+        float d = delta[i];
+        for (int p = 1; p < parts; ++p) d += delta[p * n + i];
+        x[i] = fmaf(scale[i % width], d, add ? x[i] : 0.0f);
     }
 }
 
@@ -499,6 +527,23 @@ int kipp_rmsnorm(float* x, const void* delta, int delta_dtype, int parts, const 
         if (out_dtype == KIPP_BF16) launch_rmsnorm<float, bf16_t>(x, delta, weight, out, rows, width, eps, parts, stream);
         else launch_rmsnorm<float, float>(x, delta, weight, out, rows, width, eps, parts, stream);
     }
+    return KIPP_LAUNCH_CHECK();
+}
+
+// The same with the delta's columns (float32, slabs added first) times dscale[column].
+int kipp_rmsnorm_scaled_delta(float* x, const float* delta, int parts, const float* dscale, const float* weight, void* out, int out_dtype,
+                              int rows, int width, float eps, hipStream_t stream) {
+    if (rows <= 0) return 0;
+    if (delta == nullptr || dscale == nullptr || parts <= 0) return -1;
+    if (out_dtype == KIPP_BF16) launch_rmsnorm<float, bf16_t, true>(x, delta, weight, out, rows, width, eps, parts, stream, dscale);
+    else launch_rmsnorm<float, float, true>(x, delta, weight, out, rows, width, eps, parts, stream, dscale);
+    return KIPP_LAUNCH_CHECK();
+}
+
+int kipp_scale_columns(float* x, const float* delta, int parts, size_t n, const float* scale, int width, int add, hipStream_t stream) {
+    if (n == 0) return 0;
+    if (parts <= 0 || width <= 0 || n % width) return -1;
+    hipLaunchKernelGGL(scale_columns_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, stream, x, delta, n, parts, scale, width, add);
     return KIPP_LAUNCH_CHECK();
 }
 

@@ -63,6 +63,7 @@ struct RowScale {               // sumsq == nullptr: none
 struct AddNorm {                // residual == nullptr: none
     float* residual;            // [M, N], updated in place
     const float* norm_w;        // [N]
+    const float* delta_scale;   // [N]: the product's columns times these on their way into the sum (or null)
     bf16_t* rows_out;           // [M, N] = bfloat16(residual * norm_w)
     float* sumsq_out;           // [M, stride]: ceil(N / 16) sums a row, stride as in RowScale
     int stride;
@@ -136,12 +137,16 @@ __global__ void __launch_bounds__(THREADS) gemm_skinny_kernel(
 
     // what the residual end adds to, asked for first as well (nobody writes these elements before that end does)
     const bool wide = (N & 3) == 0;                  // a lane's four columns are 16 aligned bytes
-    float res[MT][4], norm_w[4];
+    float res[MT][4], norm_w[4], delta_scale[4] = {1.0f, 1.0f, 1.0f, 1.0f};
     if (!SWIGLU && an.residual != nullptr && slice == 0) {       // the wave that will hold the tile's sums
         const int col = min(n0 + 4 * h, wide ? N - 4 : N - 1);
         if (wide) {
             const float4 w4 = *(const float4*)(an.norm_w + col);
             norm_w[0] = w4.x, norm_w[1] = w4.y, norm_w[2] = w4.z, norm_w[3] = w4.w;
+            if (an.delta_scale != nullptr) {
+                const float4 s4 = *(const float4*)(an.delta_scale + col);
+                delta_scale[0] = s4.x, delta_scale[1] = s4.y, delta_scale[2] = s4.z, delta_scale[3] = s4.w;
+            }
 #pragma unroll
             for (int mt = 0; mt < MT; ++mt) {
                 const float4 r4 = *(const float4*)(an.residual + (size_t)min(16 * mt + l16, M - 1) * N + col);
@@ -152,6 +157,7 @@ __global__ void __launch_bounds__(THREADS) gemm_skinny_kernel(
             for (int v = 0; v < 4; ++v) {
                 const int c = min(n0 + 4 * h + v, N - 1);
                 norm_w[v] = an.norm_w[c];
+                if (an.delta_scale != nullptr) delta_scale[v] = an.delta_scale[c];
 #pragma unroll
                 for (int mt = 0; mt < MT; ++mt) res[mt][v] = an.residual[(size_t)min(16 * mt + l16, M - 1) * N + c];
             }
@@ -302,7 +308,7 @@ __global__ void __launch_bounds__(THREADS) gemm_skinny_kernel(
             float x[4], ss = 0.0f;
 #pragma unroll
             for (int v = 0; v < 4; ++v) {
-                x[v] = res[mt][v] + sum[0][mt][v];
+                x[v] = fmaf(delta_scale[v], sum[0][mt][v], res[mt][v]);       // (times one: the plain sum's bits)
                 if (token < M && n + v < N) ss = fmaf(x[v], x[v], ss);
             }
             if (token < M && wide && n + 3 < N) {
@@ -468,19 +474,27 @@ int kipp_gemm_skinny_sumsq_stride(int N) { return sumsq_stride((N + 15) / 16); }
 // `residual` [M, N] (or null): the product is added to it in place (Y is not written and there is
 // one part), `rows_out` [M, N] = bfloat16(residual * norm_w) and `sumsq_out`
 // [M, kipp_gemm_skinny_sumsq_stride(N)] = every row's sums of squares of the new residual over each 16 columns
-// (M <= 16 with a residual).
-int kipp_gemm_skinny(const void* X, const void* W, float* Y, int M, int N, int K, int max_parts, int tiled,
-                     const float* sumsq, int sumsq_parts, float eps, float* residual, const float* norm_w, void* rows_out,
-                     float* sumsq_out, int x_steps_major, int rows_out_steps_major, hipStream_t stream) {
+// (M <= 16 with a residual).  `delta_scale` [N] (or null): the product's columns are multiplied by it before they are added.
+int kipp_gemm_skinny_scaled(const void* X, const void* W, float* Y, int M, int N, int K, int max_parts, int tiled,
+                            const float* sumsq, int sumsq_parts, float eps, float* residual, const float* norm_w,
+                            const float* delta_scale, void* rows_out, float* sumsq_out, int x_steps_major,
+                            int rows_out_steps_major, hipStream_t stream) {
     if (M <= 0 || N <= 0) return 0;
     if (M > 64 || K <= 0 || (K & 7) || max_parts <= 0) return -1;
     if (sumsq != nullptr && (sumsq_parts <= 0 || M > 16)) return -1;
     if (residual != nullptr && (norm_w == nullptr || rows_out == nullptr || sumsq_out == nullptr || M > 16)) return -1;
     int kw, parts;
     plan((N + 15) / 16, K, residual != nullptr ? 1 : max_parts, &kw, &parts);
-    AddNorm an = {residual, norm_w, (bf16_t*)rows_out, sumsq_out, sumsq_stride((N + 15) / 16), rows_out_steps_major};
+    AddNorm an = {residual, norm_w, delta_scale, (bf16_t*)rows_out, sumsq_out, sumsq_stride((N + 15) / 16), rows_out_steps_major};
     return launch<false>((const bf16_t*)X, (const bf16_t*)W, Y, nullptr, M, N, K, parts, kw, tiled,
                          row_scale_of(sumsq, sumsq_parts, K, eps), an, x_steps_major, 0, stream);
+}
+
+int kipp_gemm_skinny(const void* X, const void* W, float* Y, int M, int N, int K, int max_parts, int tiled,
+                     const float* sumsq, int sumsq_parts, float eps, float* residual, const float* norm_w, void* rows_out,
+                     float* sumsq_out, int x_steps_major, int rows_out_steps_major, hipStream_t stream) {
+    return kipp_gemm_skinny_scaled(X, W, Y, M, N, K, max_parts, tiled, sumsq, sumsq_parts, eps, residual, norm_w, nullptr, rows_out,
+                                   sumsq_out, x_steps_major, rows_out_steps_major, stream);
 }
 
 // W: [2 I, K] = [gate; up] (tiled: tiles of 8 gate rows over the 8 matching up rows); act: bfloat16 [M, I].
@@ -494,7 +508,7 @@ int kipp_gemm_skinny_swiglu(const void* X, const void* W, void* act, int M, int 
     if (sumsq != nullptr && (sumsq_parts <= 0 || M > 16)) return -1;
     int kw, parts;
     plan((two_inner / 2 + 7) / 8, K, 1, &kw, &parts);
-    AddNorm none = {nullptr, nullptr, nullptr, nullptr, 4, 0};
+    AddNorm none = {nullptr, nullptr, nullptr, nullptr, nullptr, 4, 0};
     return launch<true>((const bf16_t*)X, (const bf16_t*)W, nullptr, (bf16_t*)act, M, two_inner, K, 1, kw, tiled,
                         row_scale_of(sumsq, sumsq_parts, K, eps), none, x_steps_major, act_steps_major, stream);
 }

@@ -5,7 +5,7 @@
 //              weight = p / (sum of the chosen p + eps)
 //     route (grouped)  s = sigmoid(z); choice scores c = s + correction; experts in equal groups of neighbours, a group's
 //              score the sum of its two largest c; only experts of the `keep` best groups can be chosen; the `top` largest
-//              c among them; weight = s / (sum of the chosen s + eps) * scale
+//              c among them; weight = s / (sum of the chosen s + eps) * scale, or s * scale (not renormalized)
 //     sort     the (token, choice) pairs in runs of one expert each, cut into tiles of up to 16 (or 128) rows; the list of tiles
 //              is made on the device, so the host never learns the counts and the launches have a fixed shape
 //     expert   a tile's rows against its expert's matrix: out[row][n] = act(sum_k W_e[n][k] x[row][k]).  bfloat16 with K a
@@ -14,6 +14,9 @@
 //              lanes side by side) into registers while the step before is multiplied out of LDS; a tile of a few rows
 //              (single tokens) multiplies only the fragments it has, and is then bound by the read of its expert's matrix.  Else (float32, other K): a lane takes a column of a tile of 16 rows.
 //              Either way the sum over k runs in one order for every row, so a row's result does not depend on its tile
+//     gated expert  the same against an expert's [gate; up] matrix with a weight s a row of x:
+//              out[row][n] = act(s (W_gate x)[n]) * s (W_up x)[n], which is the expert applied to s x; on the matrix cores a wave's
+//              two fragments of 16 columns are the gate's and the up's of the same 16 inner columns
 //     combine  out[t] = sum_j weight[t][j] y[place of (t, j)] (+ the shared expert's result, slabs added in order)
 #include "common.h"
 #include <math.h>
@@ -104,7 +107,7 @@ moe_route_kernel(const float* __restrict__ z, int parts, size_t part_stride, int
 __global__ void __launch_bounds__(ROUTE_WAVES * KIPP_WAVE)
 moe_route_grouped_kernel(const float* __restrict__ z, int parts, size_t part_stride, int stride, const float* __restrict__ correction,
                          int32_t* __restrict__ chosen, float* __restrict__ weight, int tokens, int experts, int top, float eps,
-                         int group_count, int group_keep, float scale) {
+                         int group_count, int group_keep, float scale, int renormalize) {
     __shared__ float c_s[ROUTE_WAVES][MAX_EXPERTS];     // choice scores, then -inf for experts of groups that do not stay
     __shared__ float g_s[ROUTE_WAVES][MAX_EXPERTS];     // group scores, -inf once a group is taken
     const int wave = threadIdx.x / KIPP_WAVE, lane = threadIdx.x & (KIPP_WAVE - 1);
@@ -182,14 +185,16 @@ moe_route_grouped_kernel(const float* __restrict__ z, int parts, size_t part_str
     }
     if (live && lane < top) {
         chosen[(size_t)t * top + lane] = mine_e;
-        weight[(size_t)t * top + lane] = mine / (picked_sum + eps) * scale;
+        weight[(size_t)t * top + lane] = renormalize ? mine / (picked_sum + eps) * scale : mine * scale;
     }
 }
 
 // One workgroup sorts all pairs.  tiles: int32 [max_tiles][3] = (expert, first row, rows); rows 0 marks an unused tile.
+// `row_weight` (or null) receives every sorted row's weight.
 __global__ void __launch_bounds__(1024)
 moe_sort_kernel(const int32_t* __restrict__ chosen, int pairs, int experts, int top, int32_t* __restrict__ pair_token,
-                int32_t* __restrict__ place_of_pair, int32_t* __restrict__ tiles, int max_tiles, int tile_rows) {
+                int32_t* __restrict__ place_of_pair, int32_t* __restrict__ tiles, int max_tiles, int tile_rows,
+                const float* __restrict__ weight, float* __restrict__ row_weight) {
     __shared__ int count[MAX_EXPERTS];
     __shared__ int first[MAX_EXPERTS + 1];
     __shared__ int tile_first[MAX_EXPERTS + 1];
@@ -231,24 +236,30 @@ moe_sort_kernel(const int32_t* __restrict__ chosen, int pairs, int experts, int 
         const int at = first[e] + atomicAdd(&count[e], 1);
         pair_token[at] = p / top;
         place_of_pair[p] = at;
+        if (row_weight != nullptr) row_weight[at] = weight[p];
     }
 }
 
-// x rows are x[gather[row]] (gather null: x[row]); w: [experts][n_out][k]; out[row][n_out].
-template <typename TX, typename TW, typename TO>
+// x rows are x[gather[row]] (gather null: x[row]); w: [experts][n_out][k]; out[row][n_out].  GLU: w is [experts][2 n_out][k] =
+// [gate; up], `row_weight` (or null: one) a row's weight.
+template <typename TX, typename TW, typename TO, bool GLU>
 __global__ void __launch_bounds__(EXPERT_COLS)
-moe_expert_kernel(const TX* __restrict__ x, const int32_t* __restrict__ gather, const TW* __restrict__ w,
-                  const int32_t* __restrict__ tiles, TO* __restrict__ out, int n_out, int k, int act) {
+moe_expert_kernel(const TX* __restrict__ x, const int32_t* __restrict__ gather, const float* __restrict__ row_weight,
+                  const TW* __restrict__ w, const int32_t* __restrict__ tiles, TO* __restrict__ out, int n_out, int k, int act) {
     __shared__ float x_s[TILE_ROWS][EXPERT_KC];
     const int32_t* tile = tiles + (size_t)blockIdx.x * 3;
     const int rows = tile[2];
     if (rows == 0) return;      // uniform over the workgroup
     const int expert = tile[0], row0 = tile[1];
     const int col = blockIdx.y * EXPERT_COLS + threadIdx.x;
-    const TW* w_row = w + ((size_t)expert * n_out + (col < n_out ? col : 0)) * k;
-    float acc[TILE_ROWS];
+    const TW* w_row = w + ((size_t)expert * (GLU ? 2 : 1) * n_out + (col < n_out ? col : 0)) * k;
+    const TW* up_row = w_row + (size_t)n_out * k;
+    float acc[TILE_ROWS], up[GLU ? TILE_ROWS : 1];
 #pragma unroll
-    for (int r = 0; r < TILE_ROWS; ++r) acc[r] = 0.0f;
+    for (int r = 0; r < TILE_ROWS; ++r) {
+        acc[r] = 0.0f;
+        if (GLU) up[r] = 0.0f;
+    }
     for (int k0 = 0; k0 < k; k0 += EXPERT_KC) {
         const int kc = min(EXPERT_KC, k - k0);
         __syncthreads();
@@ -267,13 +278,27 @@ moe_expert_kernel(const TX* __restrict__ x, const int32_t* __restrict__ gather, 
                 const float wv = load_f(w_row, k0 + e);
 #pragma unroll
                 for (int r = 0; r < TILE_ROWS; ++r) acc[r] = fmaf(wv, x_s[r][e], acc[r]);
+                if (GLU) {
+                    const float uv = load_f(up_row, k0 + e);
+#pragma unroll
+                    for (int r = 0; r < TILE_ROWS; ++r) up[r] = fmaf(uv, x_s[r][e], up[r]);
+                }
             }
         }
     }
     if (col >= n_out) return;
 #pragma unroll
     for (int r = 0; r < TILE_ROWS; ++r)
-        if (r < rows) store_f(out + (size_t)(row0 + r) * n_out, col, activate(acc[r], act));
+        if (r < rows) {
+            float y;
+            if (GLU) {
+                const float s = row_weight != nullptr ? row_weight[row0 + r] : 1.0f;
+                y = activate(s * acc[r], act) * (s * up[r]);
+            } else {
+                y = activate(acc[r], act);
+            }
+            store_f(out + (size_t)(row0 + r) * n_out, col, y);
+        }
 }
 
 // The same on the matrix cores: bfloat16 x and w, K a multiple of 32, tiles of up to MFMA_ROWS rows.  A 16 x 16 x 32
@@ -287,10 +312,10 @@ union Frag {
     bf16x8 v;
 };
 
-template <typename TO>
+template <typename TO, bool GLU>
 __global__ void __launch_bounds__(MFMA_THREADS)
-moe_expert_mfma_kernel(const bf16_t* __restrict__ x, const int32_t* __restrict__ gather, const bf16_t* __restrict__ w,
-                       const int32_t* __restrict__ tiles, TO* __restrict__ out, int n_out, int k, int act) {
+moe_expert_mfma_kernel(const bf16_t* __restrict__ x, const int32_t* __restrict__ gather, const float* __restrict__ row_weight,
+                       const bf16_t* __restrict__ w, const int32_t* __restrict__ tiles, TO* __restrict__ out, int n_out, int k, int act) {
     // 64 numbers of k of every row of the tile and of every column of the workgroup, a row 144 bytes apart from the next
     // (the fragments' reads of 16 bytes a lane then spread over the banks)
     __shared__ __attribute__((aligned(16))) bf16_t a_s[MFMA_ROWS * MFMA_PITCH];
@@ -307,13 +332,13 @@ moe_expert_mfma_kernel(const bf16_t* __restrict__ x, const int32_t* __restrict__
     const int expert = tile[0], row0 = tile[1];
     const int tid = threadIdx.x;
     const int wave = tid / KIPP_WAVE, lane = tid & (KIPP_WAVE - 1), l16 = lane & 15, h = lane >> 4;
-    const int col_base = (item / gridDim.x) * MFMA_COLS;
+    const int col_base = (item / gridDim.x) * (GLU ? MFMA_COLS / 2 : MFMA_COLS);
     const int mfrags = (rows + 15) >> 4;
     // from memory, 8 threads take the 128 bytes of a row's step: thread t rows t / 8 + 32 i, bytes 16 (t % 8) ..
     const int ld_row = tid >> 3, ld_ch = tid & 7;
     // where a lane's rows begin, in numbers from x and from the expert's matrix (the launcher has checked that 32 bits hold them)
     unsigned a_src[MFMA_ROWS / 32], b_src[MFMA_COLS / 32];
-    const bf16_t* w_e = w + (size_t)expert * n_out * k;
+    const bf16_t* w_e = w + (size_t)expert * (GLU ? 2 : 1) * n_out * k;
 #pragma unroll
     for (int i = 0; i < MFMA_ROWS / 32; ++i) {
         const int r = min(ld_row + 32 * i, rows - 1);       // rows beyond the tile's read its last one and are not stored
@@ -322,7 +347,8 @@ moe_expert_mfma_kernel(const bf16_t* __restrict__ x, const int32_t* __restrict__
     }
 #pragma unroll
     for (int i = 0; i < MFMA_COLS / 32; ++i) {
-        const int c = min(col_base + ld_row + 32 * i, n_out - 1);
+        const int at = ld_row + 32 * i;         // the staged column: a wave's 32 are 16 of the gate's, then 16 of the up's
+        const int c = GLU ? min(col_base + 16 * (at >> 5) + (at & 15), n_out - 1) + (at & 16 ? n_out : 0) : min(col_base + at, n_out - 1);
         b_src[i] = (unsigned)c * (unsigned)k + 8 * ld_ch;
     }
     u32x4 a_r[MFMA_ROWS / 32], b_r[MFMA_COLS / 32];
@@ -376,6 +402,20 @@ moe_expert_mfma_kernel(const bf16_t* __restrict__ x, const int32_t* __restrict__
             }
         }
     }
+    if (GLU) {
+        const int c = col_base + wave * 16 + l16;
+#pragma unroll
+        for (int i = 0; i < MFMA_ROWS / 16; ++i)
+#pragma unroll
+            for (int v = 0; v < 4; ++v) {
+                const int r = 16 * i + 4 * h + v;
+                if (r < rows && c < n_out) {
+                    const float s = row_weight != nullptr ? row_weight[row0 + r] : 1.0f;
+                    store_f(out + (size_t)(row0 + r) * n_out, c, activate(s * acc[i][0][v], act) * (s * acc[i][1][v]));
+                }
+            }
+        return;
+    }
     const int col0 = col_base + wave * 16 * MFMA_NF;
 #pragma unroll
     for (int i = 0; i < MFMA_ROWS / 16; ++i)
@@ -393,7 +433,7 @@ moe_expert_mfma_kernel(const bf16_t* __restrict__ x, const int32_t* __restrict__
         }
 }
 
-// out[t][c] = sum_j weight[t][j] y[place[t top + j]][c] + sum of the slabs of shared[t][c]
+// out[t][c] = sum_j weight[t][j] y[place[t top + j]][c] (weight null: every weight one) + sum of the slabs of shared[t][c]
 __global__ void moe_combine_kernel(const float* __restrict__ y, const int32_t* __restrict__ place, const float* __restrict__ weight,
                                    const float* __restrict__ shared, int shared_parts, size_t shared_stride,
                                    float* __restrict__ out, int tokens, int width, int top) {
@@ -402,14 +442,14 @@ __global__ void moe_combine_kernel(const float* __restrict__ y, const int32_t* _
     const int t = (int)(i / width), c = (int)(i - (size_t)t * width);
     float acc = 0.0f;
     for (int j = 0; j < top; ++j)
-        acc = fmaf(weight[(size_t)t * top + j], y[(size_t)place[(size_t)t * top + j] * width + c], acc);
+        acc = fmaf(weight != nullptr ? weight[(size_t)t * top + j] : 1.0f, y[(size_t)place[(size_t)t * top + j] * width + c], acc);
     for (int p = 0; p < shared_parts; ++p) acc += shared[p * shared_stride + i];
     out[i] = acc;
 }
 
 extern "C" int kipp_moe_route(const float* z, int parts, int stride, int32_t* chosen, float* weight, int tokens, int experts, int top,
                               float eps, int32_t* pair_token, int32_t* place_of_pair, int32_t* tiles, int max_tiles, int tile_rows,
-                              hipStream_t stream) {
+                              float* row_weight, hipStream_t stream) {
     if (tokens <= 0) return 0;
     if (experts <= 0 || experts > MAX_EXPERTS || top <= 0 || top > MAX_TOP || top > experts || stride < experts || parts <= 0) return -1;
     const int pairs = tokens * top;
@@ -418,15 +458,15 @@ extern "C" int kipp_moe_route(const float* z, int parts, int stride, int32_t* ch
     hipLaunchKernelGGL(moe_route_kernel, dim3((tokens + ROUTE_WAVES - 1) / ROUTE_WAVES), dim3(ROUTE_WAVES * KIPP_WAVE), 0, stream, z, parts,
                        (size_t)tokens * stride, stride, chosen, weight, tokens, experts, top, eps);
     hipLaunchKernelGGL(moe_sort_kernel, dim3(1), dim3(1024), 0, stream, (const int32_t*)chosen, pairs, experts, top, pair_token,
-                       place_of_pair, tiles, max_tiles, tile_rows);
+                       place_of_pair, tiles, max_tiles, tile_rows, (const float*)weight, row_weight);
     return KIPP_LAUNCH_CHECK();
 }
 
 // The same with sigmoid scores, a correction of the choice (or none) and groups of which `group_keep` of `group_count` stay.
 extern "C" int kipp_moe_route_grouped(const float* z, int parts, int stride, const float* correction, int32_t* chosen, float* weight,
                                       int tokens, int experts, int top, float eps, int group_count, int group_keep, float scale,
-                                      int32_t* pair_token, int32_t* place_of_pair, int32_t* tiles, int max_tiles, int tile_rows,
-                                      hipStream_t stream) {
+                                      int renormalize, int32_t* pair_token, int32_t* place_of_pair, int32_t* tiles, int max_tiles, int tile_rows,
+                                      float* row_weight, hipStream_t stream) {
     if (tokens <= 0) return 0;
     if (experts <= 0 || experts > MAX_EXPERTS || top <= 0 || top > MAX_TOP || top > experts || stride < experts || parts <= 0) return -1;
     if (group_count <= 0 || experts % group_count || group_keep <= 0 || group_keep > group_count ||
@@ -436,28 +476,30 @@ extern "C" int kipp_moe_route_grouped(const float* z, int parts, int stride, con
     if (max_tiles < (pairs + tile_rows - 1) / tile_rows + (experts < pairs ? experts : pairs)) return -1;
     hipLaunchKernelGGL(moe_route_grouped_kernel, dim3((tokens + ROUTE_WAVES - 1) / ROUTE_WAVES), dim3(ROUTE_WAVES * KIPP_WAVE), 0, stream, z,
                        parts, (size_t)tokens * stride, stride, correction, chosen, weight, tokens, experts, top, eps, group_count, group_keep,
-                       scale);
+                       scale, renormalize);
     hipLaunchKernelGGL(moe_sort_kernel, dim3(1), dim3(1024), 0, stream, (const int32_t*)chosen, pairs, experts, top, pair_token,
-                       place_of_pair, tiles, max_tiles, tile_rows);
+                       place_of_pair, tiles, max_tiles, tile_rows, (const float*)weight, row_weight);
     return KIPP_LAUNCH_CHECK();
 }
 
-// `tile_rows`: the rows of the tiles that `kipp_moe_route` was asked for: 128 takes the matrix cores (bfloat16 x and w, K a multiple of 32), 16 the plain kernel.
-extern "C" int kipp_moe_expert(const void* x, int x_dtype, const int32_t* gather, const void* w, int w_dtype, const int32_t* tiles,
-                               int max_tiles, void* out, int out_dtype, int n_out, int k, int act, int tile_rows, hipStream_t stream) {
+template <bool GLU>
+static int launch_expert(const void* x, int x_dtype, const int32_t* gather, const float* row_weight, const void* w, int w_dtype,
+                         const int32_t* tiles, int max_tiles, void* out, int out_dtype, int n_out, int k, int act, int tile_rows,
+                         hipStream_t stream) {
     if (max_tiles <= 0) return 0;
     if (n_out <= 0 || k <= 0 || act < ACT_NONE || act > ACT_RELU2) return -1;
     if (tile_rows == MFMA_ROWS) {
         if (x_dtype != KIPP_BF16 || w_dtype != KIPP_BF16 || k % 32) return -2;
         // a lane's offsets into x and into an expert's matrix are 32 bits wide
-        if ((long long)max_tiles * MFMA_ROWS * k >= (1ll << 31) || (long long)n_out * k >= (1ll << 31)) return -2;
-        dim3 grid(max_tiles, (n_out + MFMA_COLS - 1) / MFMA_COLS), block(MFMA_THREADS);
+        if ((long long)max_tiles * MFMA_ROWS * k >= (1ll << 31) || (long long)(GLU ? 2 : 1) * n_out * k >= (1ll << 31)) return -2;
+        const int cols = GLU ? MFMA_COLS / 2 : MFMA_COLS;
+        dim3 grid(max_tiles, (n_out + cols - 1) / cols), block(MFMA_THREADS);
         if (out_dtype == KIPP_BF16)
-            hipLaunchKernelGGL((moe_expert_mfma_kernel<bf16_t>), grid, block, 0, stream, (const bf16_t*)x, gather, (const bf16_t*)w, tiles,
-                               (bf16_t*)out, n_out, k, act);
+            hipLaunchKernelGGL((moe_expert_mfma_kernel<bf16_t, GLU>), grid, block, 0, stream, (const bf16_t*)x, gather, row_weight,
+                               (const bf16_t*)w, tiles, (bf16_t*)out, n_out, k, act);
         else if (out_dtype == KIPP_F32)
-            hipLaunchKernelGGL((moe_expert_mfma_kernel<float>), grid, block, 0, stream, (const bf16_t*)x, gather, (const bf16_t*)w, tiles,
-                               (float*)out, n_out, k, act);
+            hipLaunchKernelGGL((moe_expert_mfma_kernel<float, GLU>), grid, block, 0, stream, (const bf16_t*)x, gather, row_weight,
+                               (const bf16_t*)w, tiles, (float*)out, n_out, k, act);
         else
             return -2;
         return KIPP_LAUNCH_CHECK();
@@ -465,14 +507,27 @@ extern "C" int kipp_moe_expert(const void* x, int x_dtype, const int32_t* gather
     if (tile_rows != TILE_ROWS) return -1;
     dim3 grid(max_tiles, (n_out + EXPERT_COLS - 1) / EXPERT_COLS), block(EXPERT_COLS);
 #define KIPP_ME(TX, TW, TO)                                                                                                  \
-    hipLaunchKernelGGL((moe_expert_kernel<TX, TW, TO>), grid, block, 0, stream, (const TX*)x, gather, (const TW*)w, tiles, \
-                       (TO*)out, n_out, k, act)
+    hipLaunchKernelGGL((moe_expert_kernel<TX, TW, TO, GLU>), grid, block, 0, stream, (const TX*)x, gather, row_weight,         \
+                       (const TW*)w, tiles, (TO*)out, n_out, k, act)
     if (x_dtype == KIPP_F32 && w_dtype == KIPP_F32 && out_dtype == KIPP_F32) KIPP_ME(float, float, float);
     else if (x_dtype == KIPP_BF16 && w_dtype == KIPP_BF16 && out_dtype == KIPP_BF16) KIPP_ME(bf16_t, bf16_t, bf16_t);
     else if (x_dtype == KIPP_BF16 && w_dtype == KIPP_BF16 && out_dtype == KIPP_F32) KIPP_ME(bf16_t, bf16_t, float);
     else return -2;
 #undef KIPP_ME
     return KIPP_LAUNCH_CHECK();
+}
+
+// `tile_rows`: the rows of the tiles that `kipp_moe_route` was asked for: 128 takes the matrix cores (bfloat16 x and w, K a multiple of 32), 16 the plain kernel.
+extern "C" int kipp_moe_expert(const void* x, int x_dtype, const int32_t* gather, const void* w, int w_dtype, const int32_t* tiles,
+                               int max_tiles, void* out, int out_dtype, int n_out, int k, int act, int tile_rows, hipStream_t stream) {
+    return launch_expert<false>(x, x_dtype, gather, nullptr, w, w_dtype, tiles, max_tiles, out, out_dtype, n_out, k, act, tile_rows, stream);
+}
+
+// The same against w [experts][2 n_out][k] = [gate; up] with a weight a sorted row (or null): out = act(s gate) * (s up).
+extern "C" int kipp_moe_expert_gated(const void* x, int x_dtype, const int32_t* gather, const float* row_weight, const void* w, int w_dtype,
+                                     const int32_t* tiles, int max_tiles, void* out, int out_dtype, int n_out, int k, int act,
+                                     int tile_rows, hipStream_t stream) {
+    return launch_expert<true>(x, x_dtype, gather, row_weight, w, w_dtype, tiles, max_tiles, out, out_dtype, n_out, k, act, tile_rows, stream);
 }
 
 extern "C" int kipp_moe_combine(const float* y, const int32_t* place, const float* weight, const float* shared, int shared_parts,

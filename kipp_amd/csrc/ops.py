@@ -147,6 +147,28 @@ def rmsnorm(x: torch.Tensor, weight: torch.Tensor, eps: float, out: torch.Tensor
     return out
 
 
+def rmsnorm_scaled_delta(x: torch.Tensor, delta: torch.Tensor, dscale: torch.Tensor, weight: torch.Tensor, eps: float,
+                         out: torch.Tensor) -> torch.Tensor:
+    """x[r, c] += dscale[c] * delta[r, c] in place (float32; `delta` may come in slabs), out = rmsnorm(x) * weight."""
+    _dev(x, delta, dscale, weight, out)
+    parts, rows, width = _slabs(delta, "rmsnorm_scaled_delta")
+    _need(x.dtype == torch.float32 and x.shape == (rows, width) and out.shape == x.shape, "rmsnorm_scaled_delta: shapes differ")
+    _need(weight.dtype == dscale.dtype == torch.float32 and weight.numel() == dscale.numel() == width, "rmsnorm_scaled_delta: float32 weight and scale [width]")
+    fn = _fn("elementwise", "kipp_rmsnorm_scaled_delta", [_c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_float, _c_ptr])
+    _check(fn(_ptr(x), _ptr(delta), parts, _ptr(dscale), _ptr(weight), _ptr(out), _code(out), rows, width, float(eps), _stream()), "rmsnorm_scaled_delta")
+    return out
+
+
+def scale_columns(delta: torch.Tensor, scale: torch.Tensor, x: torch.Tensor, add: bool = False) -> torch.Tensor:
+    """x[r, c] = scale[c] * delta[r, c] (float32; `delta` may come in slabs), or with `add` x[r, c] += that."""
+    _dev(x, delta, scale)
+    parts, rows, width = _slabs(delta, "scale_columns")
+    _need(x.dtype == scale.dtype == torch.float32 and x.shape == (rows, width) and scale.numel() == width, "scale_columns: float32 [rows, width] and a scale a column")
+    fn = _fn("elementwise", "kipp_scale_columns", [_c_ptr, _c_ptr, _c_int, _c_size, _c_ptr, _c_int, _c_int, _c_ptr])
+    _check(fn(_ptr(x), _ptr(delta), parts, x.numel(), _ptr(scale), width, int(bool(add)), _stream()), "scale_columns")
+    return x
+
+
 def residual_add(x: torch.Tensor, delta: torch.Tensor) -> torch.Tensor:
     _dev(x, delta)
     _need(x.dtype == torch.float32 and tuple(delta.shape[-2:]) == tuple(x.shape) and delta.dim() in (2, 3),
@@ -502,55 +524,60 @@ def paged_attention_wide(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.
 def latent_prepare(proj: torch.Tensor, cq_out: torch.Tensor, cache: torch.Tensor, positions: torch.Tensor,
                    seq_of_token: torch.Tensor, block_table: torch.Tensor, q_rank: int, rank: int, dr: int,
                    q_norm_w: torch.Tensor, c_norm_w: torch.Tensor, eps: float, freq: torch.Tensor, rot_dims: int,
-                   magnitude: float, write_kv: bool = True) -> torch.Tensor:
+                   magnitude: float, write_kv: bool = True, half: bool = False, kv_at: Optional[int] = None) -> torch.Tensor:
     """From the input product `proj` (float32 [tokens, >= q_rank + rank + dr], columns query latent | key/value latent |
     rotated key part | ..., or slabs of it): the query latent RMS-normed with `q_norm_w` into `cq_out`; the key/value latent
     RMS-normed with `c_norm_w` and the key part rotated at the token's position, both written as one row of rank + dr
-    numbers into the token's page of `cache` [pages, 1, page, rank + dr]."""
+    numbers into the token's page of `cache` [pages, 1, page, rank + dr].  `kv_at`: the column at which the key/value latent
+    begins (default: behind the query latent); `q_rank` 0: there is no query latent (`cq_out` and `q_norm_w` are None).
+    `half`: number i is turned with number i + rot_dims / 2, not neighbours with each other."""
+    kv_at = q_rank if kv_at is None else int(kv_at)
     _dev(proj, cq_out, cache, positions, seq_of_token, block_table, q_norm_w, c_norm_w, freq)
     for t, name in ((positions, "positions"), (seq_of_token, "seq_of_token"), (block_table, "block_table")):
         _i32(t, name)
     parts, n, stride = _slabs(proj, "latent_prepare")
-    _need(stride >= q_rank + rank + dr and cq_out.shape == (n, q_rank) and positions.numel() == n and seq_of_token.numel() == n,
+    _need(kv_at >= q_rank and stride >= kv_at + rank + dr and (q_rank == 0 or cq_out.shape == (n, q_rank)) and positions.numel() == n and seq_of_token.numel() == n,
           "latent_prepare: one row a token, projections [query latent | latent | rotated part]")
     _need(cache.dim() == 4 and cache.shape[1] == 1 and cache.shape[3] == rank + dr and block_table.dim() == 2,
           "latent_prepare: the cache is [pages, 1, page, rank + dr]")
-    _need(q_norm_w.dtype == c_norm_w.dtype == torch.float32 and q_norm_w.numel() == q_rank and c_norm_w.numel() == rank,
+    _need(c_norm_w.dtype == torch.float32 and c_norm_w.numel() == rank
+          and (q_rank == 0 or (q_norm_w.dtype == torch.float32 and q_norm_w.numel() == q_rank)),
           "latent_prepare: float32 norm weights")
     _need(rot_dims % 2 == 0 and 0 <= rot_dims <= dr and freq.dtype == torch.float32 and freq.numel() >= rot_dims // 2,
           "latent_prepare: float32 frequencies for rot_dims / 2 pairs")
     fn = _fn("latent", "kipp_latent_prepare",
              [_c_ptr, _c_int, _c_int, _c_ptr, _c_ptr, _c_float, _c_ptr, _c_int, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int,
-              _c_ptr, _c_int, _c_float] + [_c_int] * 6 + [_c_ptr])
-    _check(fn(_ptr(proj), parts, stride, _ptr(q_norm_w), _ptr(c_norm_w), float(eps), _ptr(cq_out), _code(cq_out), _ptr(cache),
+              _c_ptr, _c_int, _c_float] + [_c_int] * 8 + [_c_ptr])
+    _check(fn(_ptr(proj), parts, stride, _ptr(q_norm_w), _ptr(c_norm_w), float(eps), _ptr(cq_out), _code(cq_out if cq_out is not None else cache), _ptr(cache),
               _code(cache), _ptr(positions), _ptr(seq_of_token), _ptr(block_table), block_table.shape[1], _ptr(freq), int(rot_dims),
-              float(magnitude), n, q_rank, rank, dr, cache.shape[2], int(write_kv), _stream()), "latent_prepare")
+              float(magnitude), int(bool(half)), n, q_rank, kv_at, rank, dr, cache.shape[2], int(write_kv), _stream()), "latent_prepare")
     return cq_out
 
 
 def latent_absorb(q: torch.Tensor, w_uk: torch.Tensor, out: torch.Tensor, positions: torch.Tensor, freq: torch.Tensor,
-                  rot_dims: int, magnitude: float, heads: int, d: int, dr: int, rank: int) -> torch.Tensor:
+                  rot_dims: int, magnitude: float, heads: int, d: int, dr: int, rank: int, half: bool = False) -> torch.Tensor:
     """out [tokens, heads (rank + dr)]: every head's unrotated query part carried into the latent's space by
-    `w_uk` [heads d, rank] (q_h W_uk_h), its rotated part turned at the token's position."""
+    `w_uk` [heads d, rank] (q_h W_uk_h), its rotated part turned at the token's position (`half` as for `latent_prepare`).
+    `q`: float32 [tokens, >= heads (d + dr)] (the heads are its first columns) or slabs of it."""
     _dev(q, w_uk, out, positions, freq)
     _i32(positions, "positions")
     parts, n, stride = _slabs(q, "latent_absorb")
-    _need(stride == heads * (d + dr) and out.shape == (n, heads * (rank + dr)) and positions.numel() == n,
+    _need(stride >= heads * (d + dr) and out.shape == (n, heads * (rank + dr)) and positions.numel() == n,
           "latent_absorb: q is [tokens, heads (d + dr)], out [tokens, heads (rank + dr)]")
     _need(w_uk.shape == (heads * d, rank) and _code(w_uk) == _code(out), "latent_absorb: w_uk is [heads d, rank] in the output's type")
     _need(d * 32 + 8192 <= 64 * 1024, "latent_absorb: unrotated head size too large")
     fn = _fn("latent", "kipp_latent_absorb", [_c_ptr, _c_int, _c_ptr, _c_int, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_int, _c_float]
-             + [_c_int] * 5 + [_c_ptr])
+             + [_c_int] * 7 + [_c_ptr])
     _check(fn(_ptr(q), parts, _ptr(w_uk), _code(w_uk), _ptr(out), _code(out), _ptr(positions), _ptr(freq), int(rot_dims),
-              float(magnitude), n, heads, d, dr, rank, _stream()), "latent_absorb")
+              float(magnitude), int(bool(half)), n, heads, d, dr, rank, stride, _stream()), "latent_absorb")
     return out
 
 
 def latent_expand(lat: torch.Tensor, w_uv_t: torch.Tensor, out: torch.Tensor, heads: int, rank: int, dv: int,
-                  gate: Optional[torch.Tensor] = None, gate_at: int = 0) -> torch.Tensor:
+                  gate: Optional[torch.Tensor] = None, gate_at: int = 0, gate_each: bool = False) -> torch.Tensor:
     """out [tokens, heads dv]: head h's latent result (the first `rank` numbers of its row of `lat` [tokens, heads row])
     carried back by `w_uv_t` [heads, rank, dv], times sigmoid(gate[t, gate_at + h]) where `gate` (the float32 input
-    product, maybe in slabs) is given."""
+    product, maybe in slabs) is given; `gate_each`: a gate a number, sigmoid(gate[t, gate_at + h dv + j])."""
     _dev(lat, w_uv_t, out, gate)
     n = lat.shape[0]
     _need(lat.dim() == 2 and lat.shape[1] % heads == 0 and lat.shape[1] // heads >= rank, "latent_expand: lat is [tokens, heads row]")
@@ -560,11 +587,11 @@ def latent_expand(lat: torch.Tensor, w_uv_t: torch.Tensor, out: torch.Tensor, he
     g_parts, g_stride, g_ptr = 0, 0, None
     if gate is not None:
         g_parts, g_n, g_stride = _slabs(gate, "latent_expand")
-        _need(g_n == n and gate_at + heads <= g_stride, "latent_expand: the gate's columns lie outside the product")
+        _need(g_n == n and gate_at + heads * (dv if gate_each else 1) <= g_stride, "latent_expand: the gate's columns lie outside the product")
         g_ptr = gate.data_ptr() + 4 * gate_at
-    fn = _fn("latent", "kipp_latent_expand", [_c_ptr, _c_int, _c_int, _c_ptr, _c_int, _c_ptr, _c_int, _c_int, _c_ptr, _c_int]
+    fn = _fn("latent", "kipp_latent_expand", [_c_ptr, _c_int, _c_int, _c_ptr, _c_int, _c_ptr, _c_int, _c_int, _c_int, _c_ptr, _c_int]
              + [_c_int] * 4 + [_c_ptr])
-    _check(fn(_ptr(lat), _code(lat), lat.shape[1] // heads, _ptr(w_uv_t), _code(w_uv_t), g_ptr, g_parts, g_stride, _ptr(out),
+    _check(fn(_ptr(lat), _code(lat), lat.shape[1] // heads, _ptr(w_uv_t), _code(w_uv_t), g_ptr, g_parts, g_stride, int(bool(gate_each)), _ptr(out),
               _code(out), n, heads, rank, dv, _stream()), "latent_expand")
     return out
 
@@ -820,6 +847,107 @@ def scan_finish(o_raw: torch.Tensor, gates: torch.Tensor, gate_at: int, norm_w: 
     return out
 
 
+# --------------------------------------------------------------------------- real-gated linear recurrent unit
+
+def recurrence_state_size(width: int, taps: int) -> int:
+    """float32 numbers of a request's state: S [width], then a ring of the last `taps` inputs [taps, width]."""
+    return -(-(1 + taps) * width // 4) * 4
+
+
+def recurrence_mfma_ok(dtype: torch.dtype, size: int) -> bool:
+    """Whether the gates of parts of `size` channels run on the matrix cores (and a step of single tokens in one launch)."""
+    return dtype == torch.bfloat16 and size % 8 == 0
+
+
+def _recurrence_args(proj, columns, state, taps, width, tokens, ints, what):
+    for t, name in ints:
+        _i32(t, name)
+    _need(proj.dim() == 2 and proj.dtype == torch.float32 and proj.shape == (tokens, proj.shape[1])
+          and all(0 <= at and at + width <= proj.shape[1] for at in columns), f"{what}: proj is float32 [tokens, columns of both branches]")
+    _need(state.dim() == 2 and state.dtype == torch.float32 and state.shape[1] >= recurrence_state_size(width, taps), f"{what}: state is float32 [slots, size]")
+
+
+def recurrence_filter(proj: torch.Tensor, x_at: int, x_bias: torch.Tensor, conv_w: torch.Tensor, conv_b: torch.Tensor, state: torch.Tensor,
+                      positions: torch.Tensor, seq_of_token: torch.Tensor, q_start: torch.Tensor, q_len: torch.Tensor, slots: torch.Tensor,
+                      u: torch.Tensor) -> torch.Tensor:
+    """u [tokens, width] (float32): the columns x_at .. of the input product `proj`, with `x_bias`, through a causal filter a
+    channel (`conv_w` [taps, width], the last tap is the current token's; `conv_b`), the slot's kept inputs ahead of a portion;
+    the kept inputs are then moved on by every entry's tokens."""
+    _dev(proj, x_bias, conv_w, conv_b, state, positions, seq_of_token, q_start, q_len, slots, u)
+    tokens, width = u.shape
+    taps = conv_w.shape[0]
+    _recurrence_args(proj, (x_at,), state, taps, width, tokens, ((positions, "positions"), (seq_of_token, "seq_of_token"), (q_start, "q_start"),
+                                                                (q_len, "q_len"), (slots, "slots")), "recurrence_filter")
+    _need(conv_w.shape == (taps, width) and 1 <= taps <= 16 and conv_b.numel() == x_bias.numel() == width
+          and u.dtype == conv_w.dtype == conv_b.dtype == x_bias.dtype == torch.float32, "recurrence_filter: float32 taps [taps, width] (up to 16), biases [width]")
+    _need(positions.numel() == seq_of_token.numel() == tokens and q_start.numel() == q_len.numel() == slots.numel(), "recurrence_filter: one start, length and slot an entry")
+    fn = _fn("gated_recurrence", "kipp_recurrence_filter", [_c_ptr, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr, _c_size] + [_c_ptr] * 6
+             + [_c_int, _c_int, _c_ptr])
+    _check(fn(_ptr(proj), proj.shape[1], int(x_at), _ptr(x_bias), _ptr(conv_w), _ptr(conv_b), taps, width, _ptr(state), state.shape[1], _ptr(positions),
+              _ptr(seq_of_token), _ptr(q_start), _ptr(q_len), _ptr(slots), _ptr(u), tokens, q_start.numel(), _stream()), "recurrence_filter")
+    return u
+
+
+def _recurrence_gate_args(w, mfma, r_bias, i_bias, decay, width, what):
+    blocks = w.shape[0]
+    size = width // blocks
+    _need(width % blocks == 0 and w.shape == ((blocks, 2, size, size) if mfma else (blocks, size, 2 * size)),
+          f"{what}: the gates' matrices are [blocks, 2, size out, size in] for the matrix cores, else [blocks, size in, 2 size out]")
+    _need(not mfma or recurrence_mfma_ok(w.dtype, size), f"{what}: the matrix cores take bfloat16 and parts of a multiple of 8 channels")
+    _need(r_bias.dtype == i_bias.dtype == decay.dtype == torch.float32 and r_bias.numel() == i_bias.numel() == decay.numel() == width,
+          f"{what}: float32 biases and decay [width]")
+    return blocks
+
+
+def recurrence_gates(u: torch.Tensor, w: torch.Tensor, r_bias: torch.Tensor, i_bias: torch.Tensor, decay: torch.Tensor, terms: torch.Tensor,
+                     mfma: bool) -> torch.Tensor:
+    """terms [tokens, width, 2] (float32) = (a, sqrt(1 - a^2) i u) with r, i = sigmoid(matrix u + bias) in each of the equal parts
+    of `u` [tokens, width] and a = exp(-r decay); both gates' sums in float32 whatever the type of `w`."""
+    _dev(u, w, r_bias, i_bias, decay, terms)
+    tokens, width = u.shape
+    blocks = _recurrence_gate_args(w, mfma, r_bias, i_bias, decay, width, "recurrence_gates")
+    _need(u.dtype == terms.dtype == torch.float32 and terms.shape == (tokens, width, 2), "recurrence_gates: float32 u [tokens, width], terms [tokens, width, 2]")
+    fn = _fn("gated_recurrence", "kipp_recurrence_gates", [_c_ptr, _c_ptr, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_ptr])
+    _check(fn(_ptr(u), _ptr(w), _code(w), int(bool(mfma)), _ptr(r_bias), _ptr(i_bias), _ptr(decay), _ptr(terms), tokens, width, blocks, _stream()), "recurrence_gates")
+    return terms
+
+
+def recurrence_scan(terms: torch.Tensor, proj: torch.Tensor, y_at: int, y_bias: torch.Tensor, state: torch.Tensor, q_start: torch.Tensor,
+                    q_len: torch.Tensor, slots: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
+    """S <- terms[t, :, 0] S + terms[t, :, 1] over every entry's tokens, in order, from and into the entry's slot (S is its first
+    `width` numbers); out [tokens, width] = S gelu_tanh(proj[:, y_at:] + y_bias)."""
+    _dev(terms, proj, y_bias, state, q_start, q_len, slots, out)
+    tokens, width = out.shape
+    _recurrence_args(proj, (y_at,), state, 0, width, tokens, ((q_start, "q_start"), (q_len, "q_len"), (slots, "slots")), "recurrence_scan")
+    _need(terms.dtype == y_bias.dtype == torch.float32 and terms.shape == (tokens, width, 2) and y_bias.numel() == width
+          and q_start.numel() == q_len.numel() == slots.numel(), "recurrence_scan: float32 terms [tokens, width, 2]; one start, length and slot an entry")
+    fn = _fn("gated_recurrence", "kipp_recurrence_scan", [_c_ptr, _c_ptr, _c_int, _c_int, _c_ptr, _c_ptr, _c_size, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_ptr])
+    _check(fn(_ptr(terms), _ptr(proj), proj.shape[1], int(y_at), _ptr(y_bias), _ptr(state), state.shape[1], _ptr(q_start), _ptr(q_len), _ptr(slots),
+              _ptr(out), _code(out), q_start.numel(), width, _stream()), "recurrence_scan")
+    return out
+
+
+def recurrence_step(proj: torch.Tensor, y_at: int, x_at: int, y_bias: torch.Tensor, x_bias: torch.Tensor, conv_w: torch.Tensor, conv_b: torch.Tensor,
+                    w: torch.Tensor, r_bias: torch.Tensor, i_bias: torch.Tensor, decay: torch.Tensor, state: torch.Tensor, positions: torch.Tensor,
+                    seq_of_token: torch.Tensor, slots: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
+    """`recurrence_filter`, `recurrence_gates` (on the matrix cores), `recurrence_scan` in one launch for a batch in which every
+    entry brings one token."""
+    _dev(proj, y_bias, x_bias, conv_w, conv_b, w, r_bias, i_bias, decay, state, positions, seq_of_token, slots, out)
+    tokens, width = out.shape
+    taps = conv_w.shape[0]
+    _recurrence_args(proj, (x_at, y_at), state, taps, width, tokens, ((positions, "positions"), (seq_of_token, "seq_of_token"), (slots, "slots")), "recurrence_step")
+    blocks = _recurrence_gate_args(w, True, r_bias, i_bias, decay, width, "recurrence_step")
+    _need(conv_w.shape == (taps, width) and 1 <= taps <= 16 and conv_b.numel() == x_bias.numel() == y_bias.numel() == width
+          and conv_w.dtype == conv_b.dtype == x_bias.dtype == y_bias.dtype == torch.float32, "recurrence_step: float32 taps [taps, width] (up to 16), biases [width]")
+    _need(positions.numel() == seq_of_token.numel() == tokens and slots.numel() == tokens, "recurrence_step: every entry brings one token")
+    fn = _fn("gated_recurrence", "kipp_recurrence_step", [_c_ptr, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr,
+                                                          _c_size, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_ptr])
+    _check(fn(_ptr(proj), proj.shape[1], int(y_at), int(x_at), _ptr(y_bias), _ptr(x_bias), _ptr(conv_w), _ptr(conv_b), taps, _ptr(w), _ptr(r_bias), _ptr(i_bias),
+              _ptr(decay), _ptr(state), state.shape[1], _ptr(positions), _ptr(seq_of_token), _ptr(slots), _ptr(out), _code(out), tokens, width, blocks, _stream()),
+           "recurrence_step")
+    return out
+
+
 # --------------------------------------------------------------------------- routed feed-forward
 
 ACTIVATIONS = {"silu": 0, "relu": 1, "gelu": 2, "gelu_tanh": 3, "relu2": 4}     # relu2: the square of relu
@@ -841,12 +969,15 @@ def moe_max_tiles(tokens: int, experts: int, top: int, tile_rows: int = 16) -> i
 
 def moe_route(z: torch.Tensor, experts: int, top: int, eps: float, chosen: torch.Tensor, weight: torch.Tensor,
               pair_token: torch.Tensor, place_of_pair: torch.Tensor, tiles: torch.Tensor, tile_rows: int = 16,
-              router: str = "softmax", correction: Optional[torch.Tensor] = None, groups: Optional[tuple] = None, scale: float = 1.0):
+              router: str = "softmax", correction: Optional[torch.Tensor] = None, groups: Optional[tuple] = None, scale: float = 1.0,
+              renormalize: bool = True, row_weight: Optional[torch.Tensor] = None):
     """From router logits `z` (float32 [tokens, >= experts] or slabs): softmax over the experts, the `top` largest a token
     (`chosen`, int32 [tokens, top]) with weights p / (sum of the chosen p + eps) (`weight`, float32 [tokens, top]); then the
     pairs sorted by expert: `pair_token` [pairs] the token of every sorted row, `place_of_pair` [pairs] the row of pair
-    (token, choice), `tiles` int32 [max_tiles, 3] = (expert, first row, rows) of up to `tile_rows` rows, unused tiles with 0 rows."""
-    _dev(z, chosen, weight, pair_token, place_of_pair, tiles)
+    (token, choice), `tiles` int32 [max_tiles, 3] = (expert, first row, rows) of up to `tile_rows` rows, unused tiles with 0 rows.
+    `renormalize` False (sigmoid router): weights are the scores themselves times `scale`.  `row_weight` (float32 [pairs]) receives
+    every sorted row's weight."""
+    _dev(z, chosen, weight, pair_token, place_of_pair, tiles, row_weight)
     parts, n, stride = _slabs(z, "moe_route")
     for t, name in ((chosen, "chosen"), (pair_token, "pair_token"), (place_of_pair, "place_of_pair"), (tiles, "tiles")):
         _i32(t, name)
@@ -855,6 +986,7 @@ def moe_route(z: torch.Tensor, experts: int, top: int, eps: float, chosen: torch
           and place_of_pair.numel() == n * top and tiles.dim() == 2 and tiles.shape[1] == 3 and tiles.shape[0] >= moe_max_tiles(n, experts, top, tile_rows),
           "moe_route: output shapes")
     _need(router in ("softmax", "sigmoid"), "moe_route: router is softmax or sigmoid")
+    _need(row_weight is None or (row_weight.dtype == torch.float32 and row_weight.numel() == n * top), "moe_route: row_weight is float32 [pairs]")
     if router == "sigmoid":
         _dev(correction)
         count, keep = groups if groups is not None else (1, 1)
@@ -862,14 +994,14 @@ def moe_route(z: torch.Tensor, experts: int, top: int, eps: float, chosen: torch
         _need(count > 0 and experts % count == 0 and 0 < keep <= count and top <= keep * (experts // count),
               "moe_route: equal groups, of which at least one stays, with experts enough for a token's choice")
         fn = _fn("moe", "kipp_moe_route_grouped", [_c_ptr, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_float, _c_int, _c_int, _c_float,
-                                                   _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr])
+                                                   _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr, _c_ptr])
         _check(fn(_ptr(z), parts, stride, _ptr(correction), _ptr(chosen), _ptr(weight), n, experts, top, float(eps), int(count), int(keep), float(scale),
-                  _ptr(pair_token), _ptr(place_of_pair), _ptr(tiles), tiles.shape[0], int(tile_rows), _stream()), "moe_route")
+                  int(bool(renormalize)), _ptr(pair_token), _ptr(place_of_pair), _ptr(tiles), tiles.shape[0], int(tile_rows), _ptr(row_weight), _stream()), "moe_route")
         return chosen, weight
-    _need(correction is None and groups is None and scale == 1.0, "moe_route: correction, groups and scale belong to the sigmoid router")
-    fn = _fn("moe", "kipp_moe_route", [_c_ptr, _c_int, _c_int, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_float, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr])
+    _need(correction is None and groups is None and scale == 1.0 and renormalize, "moe_route: correction, groups, scale and weights as they are belong to the sigmoid router")
+    fn = _fn("moe", "kipp_moe_route", [_c_ptr, _c_int, _c_int, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_float, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr, _c_ptr])
     _check(fn(_ptr(z), parts, stride, _ptr(chosen), _ptr(weight), n, experts, top, float(eps), _ptr(pair_token), _ptr(place_of_pair), _ptr(tiles),
-              tiles.shape[0], int(tile_rows), _stream()), "moe_route")
+              tiles.shape[0], int(tile_rows), _ptr(row_weight), _stream()), "moe_route")
     return chosen, weight
 
 
@@ -893,13 +1025,38 @@ def moe_expert(x: torch.Tensor, gather: Optional[torch.Tensor], w: torch.Tensor,
     return out
 
 
-def moe_combine(y: torch.Tensor, place_of_pair: torch.Tensor, weight: torch.Tensor, shared: Optional[torch.Tensor], out: torch.Tensor) -> torch.Tensor:
-    """out[t] = sum_j weight[t, j] y[place_of_pair[t top + j]] + shared[t] (float32; `shared` may come in slabs or be None)."""
+def moe_expert_gated(x: torch.Tensor, gather: Optional[torch.Tensor], row_weight: Optional[torch.Tensor], w: torch.Tensor, tiles: torch.Tensor,
+                     out: torch.Tensor, activation: str, tile_rows: int = 16) -> torch.Tensor:
+    """Every tile's rows against its expert's [gate; up] matrix: out[row] = act(s gate x_row) * (s up x_row), x_row as for
+    `moe_expert`, s = row_weight[row] (None: one): what the gated expert makes of s x_row.  `w` [experts, 2 inner, k], `out`
+    [sorted rows, inner]."""
+    _dev(x, gather, row_weight, w, tiles, out)
+    _i32(tiles, "tiles")
+    if gather is not None:
+        _i32(gather, "gather")
+    inner = out.shape[1]
+    _need(w.dim() == 3 and x.dim() == 2 and x.shape[1] == w.shape[2] and out.dim() == 2 and w.shape[1] == 2 * inner and x.dtype == w.dtype,
+          "moe_expert_gated: x [rows, k], w [experts, 2 inner, k] of one type, out [rows, inner]")
+    _need(out.shape[0] == (gather.numel() if gather is not None else x.shape[0]), "moe_expert_gated: one output row a sorted row")
+    _need(row_weight is None or (row_weight.dtype == torch.float32 and row_weight.numel() == out.shape[0]), "moe_expert_gated: a float32 weight a sorted row")
+    _need(activation in ACTIVATIONS, f"moe_expert_gated: activation is one of {sorted(ACTIVATIONS)}")
+    _need(tile_rows == MOE_TILE_ROWS or (tile_rows == MOE_MFMA_ROWS and x.dtype == torch.bfloat16 and w.shape[2] % 32 == 0),
+          "moe_expert_gated: tiles of 16 rows, or of 128 for bfloat16 with K a multiple of 32")
+    fn = _fn("moe", "kipp_moe_expert_gated", [_c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_int, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr])
+    _check(fn(_ptr(x), _code(x), _ptr(gather), _ptr(row_weight), _ptr(w), _code(w), _ptr(tiles), tiles.shape[0], _ptr(out), _code(out), inner, w.shape[2],
+              ACTIVATIONS[activation], int(tile_rows), _stream()), "moe_expert_gated")
+    return out
+
+
+def moe_combine(y: torch.Tensor, place_of_pair: torch.Tensor, weight: Optional[torch.Tensor], shared: Optional[torch.Tensor], out: torch.Tensor) -> torch.Tensor:
+    """out[t] = sum_j weight[t, j] y[place_of_pair[t top + j]] + shared[t] (float32; `weight` None: every weight is one; `shared`
+    may come in slabs or be None)."""
     _dev(y, place_of_pair, weight, shared, out)
     _i32(place_of_pair, "place_of_pair")
     n, width = out.shape
-    top = weight.shape[1]
-    _need(y.dtype == weight.dtype == out.dtype == torch.float32 and y.shape == (n * top, width) and place_of_pair.numel() == n * top,
+    top = place_of_pair.numel() // max(n, 1)
+    _need(y.dtype == out.dtype == torch.float32 and y.shape == (n * top, width) and place_of_pair.numel() == n * top
+          and (weight is None or (weight.dtype == torch.float32 and weight.shape == (n, top))),
           "moe_combine: float32 y [tokens top, width], weight [tokens, top], out [tokens, width]")
     parts = 0
     if shared is not None:
@@ -1435,7 +1592,7 @@ def gemm_skinny(x: torch.Tensor, w: torch.Tensor, max_parts: int = 1, tiles: tor
     `row_scale` = (sumsq [M, P rounded up to 4], P, eps), M <= 16: row t of the
     product is multiplied by rsqrt(sum(sumsq[t, :P]) / K + eps), i.e. x holds rows
     of an RMS norm that still lack their scale.
-    `add_norm` = (residual float32 [M, N], norm_weight float32 [N]), M <= 16: the product
+    `add_norm` = (residual float32 [M, N], norm_weight float32 [N][, a float32 factor a column [N] of the product or None]), M <= 16: the product
     (in one part) is added to `residual` in place by the kernel itself and the
     call returns (rows, sumsq) instead: rows = bfloat16(residual * norm_weight)
     and sumsq [M, P rounded up to 4] with P = ceil(N / 16) sums a row: (sumsq, P, eps)
@@ -1453,23 +1610,25 @@ def gemm_skinny(x: torch.Tensor, w: torch.Tensor, max_parts: int = 1, tiles: tor
     lib = build.library("gemm_skinny")
     tiled = _tiles_ok(tiles, n, k, "gemm_skinny")
     sumsq, sumsq_parts, eps = _row_scale_args(row_scale, m, "gemm_skinny")
-    residual = norm_w = rows = sumsq_out = out = None
+    residual = norm_w = delta_scale = rows = sumsq_out = out = None
     if add_norm is None:
         parts = lib.kipp_gemm_skinny_parts(n, k, int(max_parts))
         out = torch.empty((parts, m, n), dtype=torch.float32, device=x.device)
     else:
-        residual, norm_w = add_norm
-        _dev(residual, norm_w)
+        residual, norm_w = add_norm[:2]
+        delta_scale = add_norm[2] if len(add_norm) > 2 else None
+        _dev(residual, norm_w, delta_scale)
+        _need(delta_scale is None or (delta_scale.dtype == torch.float32 and delta_scale.numel() == n), "gemm_skinny: a float32 factor a column [N]")
         _need(m <= 16 and residual.dtype == torch.float32 and residual.shape == (m, n) and residual.is_contiguous(),
               "gemm_skinny: the residual is float32 [M, N], at most 16 rows")
         _need(norm_w.dtype == torch.float32 and norm_w.numel() == n, "gemm_skinny: the norm weight is float32 [N]")
         rows = torch.empty((m, n), dtype=torch.bfloat16, device=x.device)
         sumsq_out = torch.empty((m, ((n + 15) // 16 + 3) // 4 * 4), dtype=torch.float32, device=x.device)
-    fn = _fn("gemm_skinny", "kipp_gemm_skinny",
+    fn = _fn("gemm_skinny", "kipp_gemm_skinny_scaled",
              [_c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_int, _c_float,
-              _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr])
+              _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr])
     _check(fn(_ptr(x), _ptr(tiles if tiled else w), _ptr(out), m, n, k, int(max_parts), tiled, sumsq, sumsq_parts, eps,
-              _ptr(residual), _ptr(norm_w), _ptr(rows), _ptr(sumsq_out), int(bool(x_steps_major)), int(bool(out_steps_major)),
+              _ptr(residual), _ptr(norm_w), _ptr(delta_scale), _ptr(rows), _ptr(sumsq_out), int(bool(x_steps_major)), int(bool(out_steps_major)),
               _stream()), "gemm_skinny")
     return out if add_norm is None else (rows, sumsq_out)
 

@@ -1,7 +1,7 @@
 """What every part has in common: its parameters as data, and the registries.
 
 A part class is registered under the `kind` of its spec in the registry of its
-category (mixer, feed_forward, norm, position, block).  `params(spec)` lists
+category (mixer, feed_forward, norm, position, block, scale).  `params(spec)` lists
 its tensors by local name without touching a device; the file name of a
 tensor is `spec.prefix + local_name`.
 """
@@ -22,7 +22,7 @@ class ParamSpec:
     init: Tuple[str, float] = ("normal", 0.02)
 
 
-CATEGORIES = ("mixer", "feed_forward", "norm", "position", "block", "embedding", "head", "connection")
+CATEGORIES = ("mixer", "feed_forward", "norm", "position", "block", "embedding", "head", "connection", "scale")
 _REGISTRY: Dict[str, Dict[str, type]] = {c: {} for c in CATEGORIES}
 
 

@@ -35,20 +35,42 @@ class PreNormBlock:
 
     def forward(self, x, pending, batch, cache, state):
         act = self.rt.act_dtype
-        norm1, norm2 = self.parts["mixer_norm"], self.parts["ffn_norm"]
-        rt, ffn = self.rt, self.parts["ffn"]
+        rt, norm1 = self.rt, self.parts["mixer_norm"]
         if pending is not None and not getattr(norm1, "fuses_products", False):
             pending = rt.settle(pending)
         h = norm1.forward(x, act) if pending is None else norm1.add_forward(x, pending, act)
         if not getattr(self.mixer, "takes_scaled_rows", False):
             h = rt.rows_of(h)
-        delta = self.mixer.forward(h, batch, cache, state)
+        delta = self._scaled("mixer_scale", self.mixer.forward(h, batch, cache, state))
+        if "ffn" not in self.parts:
+            return x, delta
+        norm2, ffn = self.parts["ffn_norm"], self.parts["ffn"]
         if not getattr(norm2, "fuses_products", False):
             delta = rt.settle(delta)
         h = norm2.add_forward(x, delta, act)
         if not getattr(ffn, "takes_scaled_rows", False):
             h = rt.rows_of(h)
-        return x, ffn.forward(h, batch)
+        return x, self._scaled("ffn_scale", ffn.forward(h, batch))
+
+    def _scaled(self, role, delta):
+        """A sublayer's result as it is added: times the scale in the given role, where the arrangement has one."""
+        return self.parts[role].apply(delta) if role in self.parts else delta
+
+
+@register("block", "scaled_pre_norm")
+class ScaledPreNormBlock(PreNormBlock):
+    """The pre-norm arrangement with a scale on every sublayer's result: x += mixer_scale(mixer(mixer_norm(x)));
+    x += ffn_scale(ffn(ffn_norm(x)))."""
+
+    roles = (("mixer_norm", "norm"), ("mixer", "mixer"), ("mixer_scale", "scale"),
+             ("ffn_norm", "norm"), ("ffn", "feed_forward"), ("ffn_scale", "scale"))
+
+
+@register("block", "scaled_pre_norm_mixer")
+class ScaledPreNormMixerBlock(ScaledPreNormBlock):
+    """The first half of the scaled pre-norm arrangement alone: a layer without a feed-forward."""
+
+    roles = (("mixer_norm", "norm"), ("mixer", "mixer"), ("mixer_scale", "scale"))
 
 
 @register("block", "post_norm")

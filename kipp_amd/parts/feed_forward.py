@@ -100,7 +100,9 @@ class GatedMLP:
 @register("feed_forward", "routed_mlp")
 class RoutedMLP:
     """A mixture of experts (`RoutedMLPSpec`): delta = sum over a token's `top` experts of weight_e W_down_e act(W_up_e x),
-    plus a shared expert of the same form.  The router's logits come out of a product in float32; choice, sort and the
+    plus a shared expert of the same form; or with a gate W_down_e (act(W_gate_e x) * (W_up_e x)), the weight then maybe on the
+    expert's input (a factor on a row commutes with the two products in front of the activation, so it is applied to their
+    float32 sums: act(s gate) * (s up)).  The router's logits come out of a product in float32; choice, sort and the
     experts' products over the sorted rows are kernels whose launches have a fixed shape (the list of row tiles is made on
     the device), so nothing is read back and a step of single tokens can be recorded."""
 
@@ -119,9 +121,13 @@ class RoutedMLP:
         if getattr(s, "correction_name", None) is not None:
             p[s.correction_name] = ParamSpec((s.experts,), "float", ("normal", 0.1))
         for e in range(s.experts):
+            if s.gate_name is not None:
+                p[s.expert_prefix.format(e) + s.gate_name] = ParamSpec((s.expert_size, s.hidden_size))
             p[s.expert_prefix.format(e) + up] = ParamSpec((s.expert_size, s.hidden_size))
             p[s.expert_prefix.format(e) + down] = ParamSpec((s.hidden_size, s.expert_size))
         if s.shared_size is not None:
+            if s.gate_name is not None:
+                p[s.shared_prefix + s.gate_name] = ParamSpec((s.shared_size, s.hidden_size))
             p[s.shared_prefix + up] = ParamSpec((s.shared_size, s.hidden_size))
             p[s.shared_prefix + down] = ParamSpec((s.hidden_size, s.shared_size))
         return p
@@ -144,13 +150,20 @@ class RoutedMLP:
             router = torch.cat([router, torch.zeros((pad, router.shape[1]), dtype=router.dtype, device=router.device)], dim=0)
         self.w_router = self.rt.weight(router.contiguous())
         ups = [tensors[s.expert_prefix.format(e) + up] for e in range(s.experts)]
+        if s.gate_name is not None:         # [gate; up], rows under each other
+            gates = [tensors[s.expert_prefix.format(e) + s.gate_name] for e in range(s.experts)]
+            ups = [torch.cat([g, u] if g.dtype == u.dtype else [g.float(), u.float()], dim=0) for g, u in zip(gates, ups)]
         downs = [tensors[s.expert_prefix.format(e) + down] for e in range(s.experts)]
         if len({t.dtype for t in ups + downs}) > 1:
             ups, downs = [t.float() for t in ups], [t.float() for t in downs]
-        self.w_up = torch.stack(ups).contiguous()           # [experts, inner, hidden]
+        self.w_up = torch.stack(ups).contiguous()           # [experts, inner, hidden], or [experts, 2 inner, hidden] with a gate
         self.w_down = torch.stack(downs).contiguous()       # [experts, hidden, inner]
         if s.shared_size is not None:
-            self.w_shared_up = self.rt.weight(tensors[s.shared_prefix + up])
+            shared_up = tensors[s.shared_prefix + up]
+            if s.gate_name is not None:
+                gate = tensors[s.shared_prefix + s.gate_name]
+                shared_up = torch.cat([gate, shared_up] if gate.dtype == shared_up.dtype else [gate.float(), shared_up.float()], dim=0).contiguous()
+            self.w_shared_up = self.rt.weight(shared_up)
             self.w_shared_down = self.rt.weight(tensors[s.shared_prefix + down])
 
     def forward(self, x, batch=None):
@@ -166,17 +179,23 @@ class RoutedMLP:
         # bfloat16 experts whose two contractions are multiples of 32 run on the matrix cores, in tiles of 128 rows
         tile_rows = ops.moe_tile_rows(self.w_up.dtype, s.hidden_size, s.expert_size)
         tiles = torch.empty((ops.moe_max_tiles(n, s.experts, s.top, tile_rows), 3), dtype=torch.int32, device=dev)
+        # the weights in the order of the sorted rows, for experts that are given weighed inputs
+        row_weight = rt.empty((pairs,), torch.float32) if s.weigh_input else None
         if s.router == "sigmoid":
             ops.moe_route(z, s.experts, s.top, s.weight_eps, chosen, weight, pair_token, place, tiles, tile_rows=tile_rows, router="sigmoid",
-                          correction=self.correction, groups=s.groups, scale=s.route_scale)
+                          correction=self.correction, groups=s.groups, scale=s.route_scale, renormalize=s.renormalize, row_weight=row_weight)
         else:
-            ops.moe_route(z, s.experts, s.top, s.weight_eps, chosen, weight, pair_token, place, tiles, tile_rows=tile_rows)
+            ops.moe_route(z, s.experts, s.top, s.weight_eps, chosen, weight, pair_token, place, tiles, tile_rows=tile_rows, row_weight=row_weight)
         if x.dtype != self.w_up.dtype:
             x = ops.cast(x, rt.empty(x.shape, self.w_up.dtype))
-        inner = ops.moe_expert(x, pair_token, self.w_up, tiles, rt.empty((pairs, s.expert_size), self.w_up.dtype), s.activation, tile_rows=tile_rows)
+        inner = rt.empty((pairs, s.expert_size), self.w_up.dtype)
+        if s.gate_name is not None:
+            ops.moe_expert_gated(x, pair_token, row_weight, self.w_up, tiles, inner, s.activation, tile_rows=tile_rows)
+        else:
+            ops.moe_expert(x, pair_token, self.w_up, tiles, inner, s.activation, tile_rows=tile_rows)
         y = ops.moe_expert(inner, None, self.w_down, tiles, rt.empty((pairs, s.hidden_size), torch.float32), tile_rows=tile_rows)
         shared = None
         if s.shared_size is not None:
-            mid = ops.activate(rt.linear(x, self.w_shared_up, slabs=True), rt.empty((n, s.shared_size), rt.act_dtype), s.activation)
+            mid = ops.activate(rt.linear(x, self.w_shared_up, slabs=True), rt.empty((n, s.shared_size), rt.act_dtype), s.activation, glu=s.gate_name is not None)
             shared = rt.linear(mid, self.w_shared_down, slabs=True)
-        return ops.moe_combine(y, place, weight, shared, rt.empty((n, s.hidden_size), torch.float32))
+        return ops.moe_combine(y, place, None if s.weigh_input else weight, shared, rt.empty((n, s.hidden_size), torch.float32))

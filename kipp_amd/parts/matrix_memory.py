@@ -157,6 +157,7 @@ class SSD:
     decay a token and head, keys B and queries C that the heads of a group share, and values dt u."""
 
     graph_safe = True   # forward launches kernels only: no host reads, no data-dependent launches
+    takes_scaled_rows = True
 
     def __init__(self, spec, runtime):
         self.spec = spec

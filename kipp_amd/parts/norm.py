@@ -16,7 +16,7 @@ parts that do not say they take them.
 """
 from __future__ import annotations
 
-from ..runtime import Deferred, Pending, WeightedDelta
+from ..runtime import ColumnScaled, Deferred, Pending, WeightedDelta
 from .base import ParamSpec, register
 
 
@@ -48,6 +48,13 @@ class RMSNorm:
         return self.rt.ops.rmsnorm(x, self.weight, self.spec.eps, self.rt.empty(x.shape, out_dtype))
 
     def add_forward(self, x, delta, out_dtype):
+        if isinstance(delta, ColumnScaled):
+            scale, delta = delta.scale, delta.delta
+            if isinstance(delta, Deferred) and out_dtype == self.rt.act_dtype:
+                fused = self.rt.product_add_norm(delta, x, self.weight, self.spec.eps, scale=scale)
+                if fused is not None:
+                    return fused
+            return self.rt.ops.rmsnorm_scaled_delta(x, self.rt.settle(delta), scale, self.weight, self.spec.eps, self.rt.empty(x.shape, out_dtype))
         if isinstance(delta, Deferred):       # a product not launched yet: add and norm ride on it where they can
             fused = self.rt.product_add_norm(delta, x, self.weight, self.spec.eps) if out_dtype == self.rt.act_dtype else None
             if fused is not None:

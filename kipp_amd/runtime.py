@@ -134,6 +134,23 @@ class WeightedDelta(Pending):
         return out
 
 
+class ColumnScaled(Pending):
+    """A delta whose columns are multiplied by a vector before it is added: scale * delta, `delta` a tensor, slabs of one or
+    another `Pending`, `scale` float32 [width].  A norm carries it out in its own kernel (or in the product's that makes the
+    delta); `add_to(x)` adds it to the residual stream, `run()` gives it as a tensor."""
+    __slots__ = ("rt", "delta", "scale")
+
+    def __init__(self, rt, delta, scale):
+        self.rt, self.delta, self.scale = rt, delta, scale
+
+    def add_to(self, x):
+        return self.rt.ops.scale_columns(self.rt.settle(self.delta), self.scale, x, add=True)
+
+    def run(self):
+        delta = self.rt.settle(self.delta)
+        return self.rt.ops.scale_columns(delta, self.scale, self.rt.empty(tuple(delta.shape[-2:]), torch.float32))
+
+
 class Runtime:
     FUSE_NORM_X_BYTES = 40e6    # most bytes of X the workgroups of an unsplit product may read together for the fused norm to pay
 
@@ -218,8 +235,8 @@ class Runtime:
             return h
         return self.ops.scale_rows(h.rows, h.sumsq, h.parts, h.eps, self.empty(h.rows.shape, torch.bfloat16), steps_major=h.steps_major)
 
-    def product_add_norm(self, delta: Deferred, x: torch.Tensor, norm_weight: torch.Tensor, eps: float):
-        """x += delta's product, in the product's own kernel, which also prepares the
+    def product_add_norm(self, delta: Deferred, x: torch.Tensor, norm_weight: torch.Tensor, eps: float, scale: torch.Tensor | None = None):
+        """x += delta's product (its columns times `scale`, if given), in the product's own kernel, which also prepares the
         RMS norm of the new x: returns ScaledRows (None if this product has no such
         kernel: the caller then runs it and norms as usual)."""
         w = delta.w
@@ -237,7 +254,7 @@ class Runtime:
         if self.ops.gemm_skinny_parts(n_out, k, most) > 1 and ((n_out + 15) // 16) * rows * k * 2 > self.fuse_norm_x_bytes:
             return None
         major = self.steps_major_rows and n_out % 32 == 0 and rows > 1       # one row is one run either way
-        rows_out, sumsq = self.ops.gemm_skinny(delta.x, w.rows, tiles=w.tiles, add_norm=(x, norm_weight),
+        rows_out, sumsq = self.ops.gemm_skinny(delta.x, w.rows, tiles=w.tiles, add_norm=(x, norm_weight, scale),
                                                x_steps_major=delta.x_steps_major, out_steps_major=major)
         return ScaledRows(rows_out, sumsq, (w.shape[0] + 15) // 16, eps, steps_major=major)
 
