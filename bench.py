@@ -350,6 +350,30 @@ def zivazen_config(qwen: dict, layers: int, kind: str) -> dict:
     return {"architecture": "Zivazen", "vocab": qwen["vocab_size"], "width": width, "norm": {"eps": 1e-6}, "layers": made}
 
 
+def bipazen_config(qwen: dict, layers: int, kind: str) -> dict:
+    """A Bipazen configuration with the layer sizes of a Qwen3 shape (width, vocabulary) and `layers` layers of one kind, so
+    that every mechanism's kernels stand beside their like alone: "mamba2" (width / 64 heads of 64 with a state of 128 and a
+    filter of 4 taps: Zivazen's state space layer), "rglru" (as wide as the model, in blocks of 256 channels, 4 taps), "latent"
+    (16 heads over a cached row of 192 + 64 numbers, every key seen: Rerizen's latent without its window), or "mixed" (mamba2,
+    rglru, rglru, latent in turn, the second time round with the first round's weights).  Every layer has the routed
+    feed-forward: 32 gated experts of a quarter of the dense inner size, 4 a token, so that a token multiplies as much as in the
+    dense layer."""
+    width, ff = qwen["hidden_size"], qwen["intermediate_size"]
+    mamba2 = {"heads": width // 64, "vdim": 64, "state": 128, "groups": 1, "conv": 4, "norm_groups": 1}
+    rglru = {"width": width, "blocks": width // 256, "conv": 4}
+    latent = {"heads": 16, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 192, "scale": 192 ** -0.5, "rot": {"base": 10000.0, "dims": 64}}
+    moe = {"kind": "moe", "router": {"experts": 32, "top": 4}, "expert": {"ff": ff // 4}}
+    mixers = {"mamba2": ("mamba2", mamba2), "rglru": ("rglru", rglru), "latent": ("latent_attention", latent)}
+    order = ["mamba2", "rglru", "rglru", "latent"] if kind == "mixed" else [kind]
+    made = []
+    for i in range(layers):
+        name, mixer = mixers[order[i % len(order)]]
+        made.append({"type": name, "mixer": json.loads(json.dumps(mixer)), "mlp": json.loads(json.dumps(moe))})
+        if kind == "mixed" and i >= len(order):
+            made[-1]["weights_of"] = i % len(order)
+    return {"architecture": "Bipazen", "vocab": qwen["vocab_size"], "width": width, "norm": {"eps": 1e-6}, "max_position": 8192, "layers": made}
+
+
 def design_points(config, args, label):
     """Prefill of one 2,048-token prompt and decode steps at two batch sizes behind such prompts, for one model made
     with random weights: milliseconds, tokens a second, and what the kernels ran as (recorded steps, library products,
@@ -459,6 +483,29 @@ def zivazen_bench(args) -> int:
     return 0
 
 
+def bipazen_bench(args) -> int:
+    """`--design bipazen`: the Bipazen design beside Qwen3 and beside the layers that are closest to its own (Rerizen's latent
+    attention, Zivazen's state space layer beside its window attention, Bebulorn's routed feed-forward) at equal layer sizes, a
+    few layers of each, random weights: one model for each of its mixers alone, and one with all of them in turn."""
+    from kipp_amd.config import shape_config
+    layers = args.layers or 4
+    kinds = args.design_kinds if args.design_kinds != DESIGN_KINDS_DEFAULT else "mamba2,rglru,latent,mixed"
+    sizes = {}
+    for shape in [s for s in args.design_shapes.split(",") if s]:
+        qwen = shape_config(shape)
+        qwen["num_hidden_layers"] = layers
+        sizes[shape] = {"qwen3": design_points(qwen, args, f"{shape} qwen3"),
+                        "rerizen_latent": design_points(rerizen_config(qwen, layers, "latent"), args, f"{shape} rerizen, latent"),
+                        "zivazen_parallel": design_points(zivazen_config(qwen, layers, "parallel"), args, f"{shape} zivazen, parallel"),
+                        "bebulorn_moe": design_points(bebulorn_config(qwen, layers, "moe"), args, f"{shape} bebulorn, moe")}
+        for kind in [k for k in kinds.split(",") if k]:
+            sizes[shape][f"bipazen_{kind}"] = design_points(bipazen_config(qwen, layers, kind), args, f"{shape} bipazen, {kind}")
+    print(json.dumps({"metric": "prefill and decode of the Bipazen design beside Qwen3 and the closest layers of other designs at equal layer sizes (bf16, random weights)",
+                      "design": "bipazen", "layers": layers, "prompt_tokens": args.prompt, "steps": args.steps,
+                      "unit": "ms and tok/s", "n_gpus": 1, "dtype": "bf16", "data": "synthetic", "sizes": sizes}), flush=True)
+    return 0
+
+
 def design_bench(args) -> int:
     """`--design tobinex`: the Tobinex design beside Qwen3 at equal layer sizes (both with every key kept, and Tobinex
     once more with a window of 1,024 keys behind 4 kept ones), a few layers of each, random weights."""
@@ -498,12 +545,12 @@ def main():
     ap.add_argument("--no-c-host", action="store_true", help="leave out the points measured through the C host")
     ap.add_argument("--products", choices=["default", "own", "auto", "library"], default="default",
                     help="products of many rows (prompt portions): the runtime's default, our kernel only, the fastest of ours and the library's, the library's")
-    ap.add_argument("--design", choices=["tobinex", "rerizen", "bebulorn", "zivazen"], default=None,
+    ap.add_argument("--design", choices=["tobinex", "rerizen", "bebulorn", "zivazen", "bipazen"], default=None,
                     help="instead of the default workload: this design beside Qwen3 at equal layer sizes (prefill and decode, a few layers)")
     ap.add_argument("--design-shapes", default="qwen3-4b,qwen3-8b", help="the Qwen3 shapes whose layer sizes --design takes")
     ap.add_argument("--design-kinds", default=DESIGN_KINDS_DEFAULT,
-                    help="--design rerizen, bebulorn or zivazen: the models that are measured, one mechanism each or all in turn "
-                         "(bebulorn: attention,lightning,delta,moe,mixed; zivazen: attention,attention_narrow,parallel,moe,mixed)")
+                    help="--design rerizen, bebulorn, zivazen or bipazen: the models that are measured, one mechanism each or all in turn "
+                         "(bebulorn: attention,lightning,delta,moe,mixed; zivazen: attention,attention_narrow,parallel,moe,mixed; bipazen: mamba2,rglru,latent,mixed)")
     args = ap.parse_args()
     if args.gpus != 1:
         print(f"bench: this engine runs on one GPU; --gpus {args.gpus} is not supported")
@@ -512,6 +559,8 @@ def main():
         return rerizen_bench(args)
     if args.design == "bebulorn":
         return bebulorn_bench(args)
+    if args.design == "bipazen":
+        return bipazen_bench(args)
     if args.design == "zivazen":
         return zivazen_bench(args)
     if args.design:
