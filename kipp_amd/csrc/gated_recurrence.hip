@@ -26,20 +26,30 @@ typedef __attribute__((ext_vector_type(4))) uint32_t u32x4;
 union Frag {
     u32x4 u;
     bf16x8 v;
-    bf16_t e[8];
+    __bf16 e[8];
 };
 
-__device__ __forceinline__ float sigmoid_f(float z) { return 1.0f / (1.0f + expf(-z)); }
+// The reciprocal and the root within an ulp, in one instruction each: enough for everything below.
+__device__ __forceinline__ float sigmoid_f(float z) { return __builtin_amdgcn_rcpf(1.0f + expf(-z)); }
 // 0.5 z (1 + tanh(w)) = z / (1 + e^(-2 w))
 __device__ __forceinline__ float gelu_tanh_f(float z) {
     const float w = 0.79788456080286535588f * (z + 0.044715f * z * z * z);
-    return z / (1.0f + expf(-2.0f * w));
+    return z * __builtin_amdgcn_rcpf(1.0f + expf(-2.0f * w));
+}
+
+// 1 - e^x for x <= 0: near zero the power series of e^x - 1 (nine terms: below half an ulp for x > -1/2), else the difference.
+__device__ __forceinline__ float one_minus_exp(float x, float exp_x) {
+    float s = 1.0f + x * (1.0f / 9.0f);
+#pragma unroll
+    for (int k = 8; k >= 2; --k) s = fmaf(s * x, 1.0f / (float)k, 1.0f);
+    return x > -0.5f ? -x * s : 1.0f - exp_x;
 }
 
 // (a, sqrt(1 - a^2) i u) from the two gates' sums (biases added).
 __device__ __forceinline__ float2 recurrence_terms(float zr, float zi, float decay, float u) {
     const float log_a = -decay * sigmoid_f(zr);
-    return make_float2(expf(log_a), sqrtf(-expm1f(2.0f * log_a)) * (sigmoid_f(zi) * u));
+    const float a = expf(log_a);
+    return make_float2(a, __builtin_amdgcn_sqrtf(one_minus_exp(2.0f * log_a, a * a)) * (sigmoid_f(zi) * u));
 }
 
 struct Filter {
@@ -51,29 +61,58 @@ struct Filter {
     int taps, width;
 };
 
-// u of token row t at position p, channel c; `first` is the row of its entry's first token, `ring` the slot's kept inputs.
-__device__ __forceinline__ float filter_at(const Filter& f, int t, int first, int p, const float* __restrict__ ring, int c) {
-    float y = f.b[c];
-    const float xb = f.x_bias[c];
-    for (int j = 0; j < f.taps; ++j) {
-        const int back = f.taps - 1 - j;
-        float in = 0.0f;
-        if (t - back >= first) in = f.proj[(size_t)(t - back) * f.stride + f.x_at + c] + xb;
-        else if (p - back >= 0) in = ring[(size_t)((p - back) % f.taps) * f.width + c];
-        y = fmaf(f.w[(size_t)j * f.width + c], in, y);
+// One channel's filter in registers.  TAPS: the number of taps if the build knows it, 0: whatever `f.taps` says.
+template <int TAPS>
+struct Channel {
+    static constexpr int MOST = TAPS > 0 ? TAPS : MAX_TAPS;
+    float w[MOST], b, xb;
+    int c, taps;
+    __device__ __forceinline__ Channel(const Filter& f, int channel) {
+        c = channel;
+        taps = TAPS > 0 ? TAPS : f.taps;
+        b = f.b[c];
+        xb = f.x_bias[c];
+#pragma unroll
+        for (int j = 0; j < MOST; ++j) w[j] = j < taps ? f.w[(size_t)j * f.width + c] : 0.0f;
     }
-    return y;
-}
+    // u of token row t at position p; `first` is the row of its entry's first token, `ring` the slot's kept inputs.
+    __device__ __forceinline__ float at(const Filter& f, int t, int first, int p, const float* __restrict__ ring) const {
+        const int turn = p % taps;
+        float in[MOST];
+#pragma unroll
+        for (int j = 0; j < MOST; ++j) {        // every load is asked for before the first is used
+            const int back = taps - 1 - j;
+            in[j] = 0.0f;
+            if (j < taps) {
+                if (t - back >= first) in[j] = f.proj[(size_t)(t - back) * f.stride + f.x_at + c] + xb;
+                else if (p - back >= 0) in[j] = ring[(size_t)(turn - back + (turn < back ? taps : 0)) * f.width + c];
+            }
+        }
+        float y = b;
+#pragma unroll
+        for (int j = 0; j < MOST; ++j)
+            if (j < taps) y = fmaf(w[j], in[j], y);
+        return y;
+    }
+};
 
+#define FILTER_TOKENS 8     // tokens a thread takes: its channel's taps are read once for them
+
+template <int TAPS>
 __global__ void __launch_bounds__(THREADS)
 filter_kernel(Filter f, const float* __restrict__ state, size_t state_stride, const int32_t* __restrict__ positions,
               const int32_t* __restrict__ seq_of_token, const int32_t* __restrict__ q_start, const int32_t* __restrict__ slots,
-              float* __restrict__ u) {
-    const int t = blockIdx.x, c = blockIdx.y * THREADS + threadIdx.x;
+              float* __restrict__ u, int tokens) {
+    const int c = blockIdx.y * THREADS + threadIdx.x;
     if (c >= f.width) return;
-    const int entry = seq_of_token[t];
-    const float* ring = state + (size_t)slots[entry] * state_stride + f.width;
-    u[(size_t)t * f.width + c] = filter_at(f, t, q_start[entry], positions[t], ring, c);
+    const Channel<TAPS> channel(f, c);
+    const int t0 = blockIdx.x * FILTER_TOKENS, t1 = min(t0 + FILTER_TOKENS, tokens);
+#pragma unroll(TAPS > 0 ? 4 : 1)
+    for (int t = t0; t < t1; ++t) {
+        const int entry = seq_of_token[t];
+        const float* ring = state + (size_t)slots[entry] * state_stride + f.width;
+        u[(size_t)t * f.width + c] = channel.at(f, t, q_start[entry], positions[t], ring);
+    }
 }
 
 // The slot's ring after a portion: its last `taps` inputs (as many as the portion has) at their positions' places.
@@ -131,13 +170,13 @@ gates_kernel(const float* __restrict__ u, const TW* __restrict__ w, const float*
     }
 }
 
-// u as three bfloat16 numbers: the nearest, the nearest to what is left, and once more.
-__device__ __forceinline__ void split3(float v, bf16_t& hi, bf16_t& mid, bf16_t& lo) {
-    hi = f32_to_bf16(v);
-    v -= bf16_to_f32(hi);
-    mid = f32_to_bf16(v);
-    v -= bf16_to_f32(mid);
-    lo = f32_to_bf16(v);
+// u as three bfloat16 numbers: the nearest, the nearest to what is left, and once more (the conversions of the hardware).
+__device__ __forceinline__ void split3(float v, __bf16& hi, __bf16& mid, __bf16& lo) {
+    hi = (__bf16)v;
+    v -= (float)hi;
+    mid = (__bf16)v;
+    v -= (float)mid;
+    lo = (__bf16)v;
 }
 
 // ---- the gates on the matrix cores: bfloat16 matrices [blocks][2][size out][size in], size a multiple of 8.  A workgroup
@@ -229,21 +268,26 @@ gates_mfma_kernel(const float* __restrict__ u, const bf16_t* __restrict__ w, con
     }
 }
 
-// ---- the walk: a workgroup takes (entry, 16 channels); 64 tokens of terms come through LDS at a time, 16 lanes walk them in
-// order while the next 64 are on their way into registers, then every thread multiplies by the other branch and writes.
+// ---- the walk: a workgroup takes (entry, 16 channels).  Its first wave walks a run of 192 tokens out of LDS in order (16
+// lanes, a channel each), while the other three bring the next run from registers into LDS, ask memory for the one after it, and
+// multiply the run before by the other branch and write it: one barrier a run.
 #define SCAN_CH 16
-#define SCAN_T 64
-#define SCAN_N (SCAN_T * SCAN_CH / THREADS)
+#define SCAN_T 192
+#define SCAN_MOVERS (THREADS - KIPP_WAVE)
+#define SCAN_STEP (SCAN_MOVERS / SCAN_CH)       // tokens the movers take side by side
+#define SCAN_N (SCAN_T / SCAN_STEP)
 
 template <typename TO>
 __global__ void __launch_bounds__(THREADS)
 scan_kernel(const float2* __restrict__ terms, const float* __restrict__ proj, int stride, int y_at, const float* __restrict__ y_bias,
             float* __restrict__ state, size_t state_stride, const int32_t* __restrict__ q_start, const int32_t* __restrict__ q_len,
             const int32_t* __restrict__ slots, TO* __restrict__ out, int width) {
-    __shared__ float2 in_s[SCAN_T * SCAN_CH];
-    __shared__ float s_s[SCAN_T * SCAN_CH];
+    __shared__ float2 in_s[2][SCAN_T * SCAN_CH];
+    __shared__ float s_s[2][SCAN_T * SCAN_CH];
     const int entry = blockIdx.y;
-    const int ch = threadIdx.x & (SCAN_CH - 1), tt = threadIdx.x / SCAN_CH;
+    const bool walker = threadIdx.x < KIPP_WAVE;
+    const int mover = threadIdx.x - KIPP_WAVE;
+    const int ch = (walker ? threadIdx.x : mover) & (SCAN_CH - 1), tt = mover / SCAN_CH;
     const int c = min(blockIdx.x * SCAN_CH + ch, width - 1);
     const bool live = blockIdx.x * SCAN_CH + ch < width;
     const int first = q_start[entry], n = q_len[entry];
@@ -252,51 +296,72 @@ scan_kernel(const float2* __restrict__ terms, const float* __restrict__ proj, in
     float S = walks ? *s_at : 0.0f;
     const float yb = y_bias[c];
     float2 in_r[SCAN_N];
-    float y_r[SCAN_N], y_now[SCAN_N];
+    float y_r[SCAN_N];
     auto fetch = [&](int t0) {
 #pragma unroll
         for (int j = 0; j < SCAN_N; ++j) {
-            const int t = t0 + tt + j * (THREADS / SCAN_CH);
-            if (t < n) {
-                in_r[j] = terms[(size_t)(first + t) * width + c];
-                y_r[j] = proj[(size_t)(first + t) * stride + y_at + c];
-            }
+            const int t = t0 + tt + j * SCAN_STEP;
+            if (t < n) in_r[j] = terms[(size_t)(first + t) * width + c];
         }
     };
-    fetch(0);
-    for (int t0 = 0; t0 < n; t0 += SCAN_T) {
-        const int m = min(SCAN_T, n - t0);
-        // (what the walkers read last round lies behind the barrier in front of the write-out)
+    auto store = [&](float2* to) {
 #pragma unroll
-        for (int j = 0; j < SCAN_N; ++j) {
-            in_s[threadIdx.x + j * THREADS] = in_r[j];
-            y_now[j] = y_r[j];
-        }
-        __syncthreads();
-        fetch(t0 + SCAN_T);
-        if (walks) {
-            int t = 0;
-            for (; t + 8 <= m; t += 8) {
-                float2 v[8];
+        for (int j = 0; j < SCAN_N; ++j) to[(tt + j * SCAN_STEP) * SCAN_CH + ch] = in_r[j];
+    };
+    const int runs = (n + SCAN_T - 1) / SCAN_T;
+    if (!walker) {
+        fetch(0);
+        store(in_s[0]);
+        fetch(SCAN_T);
+    }
+    for (int run = 0; run <= runs; ++run) {
+        __syncthreads();        // run `run` lies in LDS, run `run - 1` has been walked
+        if (walker) {
+            if (walks && run < runs) {
+                const float2* in = in_s[run & 1] + ch;
+                float* to = s_s[run & 1] + ch;
+                const int m = min(SCAN_T, n - run * SCAN_T);
+                float2 v[8], next[8];
 #pragma unroll
-                for (int e = 0; e < 8; ++e) v[e] = in_s[(t + e) * SCAN_CH + ch];
+                for (int e = 0; e < 8; ++e) v[e] = in[e * SCAN_CH];
+                int t = 0;
+                for (; t + 8 <= m; t += 8) {
+                    const int ahead = min(t + 8, SCAN_T - 8);       // (beyond the run: read again and dropped)
 #pragma unroll
-                for (int e = 0; e < 8; ++e) {
-                    S = fmaf(v[e].x, S, v[e].y);
-                    s_s[(t + e) * SCAN_CH + ch] = S;
+                    for (int e = 0; e < 8; ++e) next[e] = in[(ahead + e) * SCAN_CH];
+#pragma unroll
+                    for (int e = 0; e < 8; ++e) {
+                        S = fmaf(v[e].x, S, v[e].y);
+                        to[(t + e) * SCAN_CH] = S;
+                    }
+#pragma unroll
+                    for (int e = 0; e < 8; ++e) v[e] = next[e];
+                }
+                for (; t < m; ++t) {
+                    const float2 one = in[t * SCAN_CH];
+                    S = fmaf(one.x, S, one.y);
+                    to[t * SCAN_CH] = S;
                 }
             }
-            for (; t < m; ++t) {
-                const float2 v = in_s[t * SCAN_CH + ch];
-                S = fmaf(v.x, S, v.y);
-                s_s[t * SCAN_CH + ch] = S;
-            }
-        }
-        __syncthreads();
+        } else {
+            if (run > 0) {      // the run before: its other branch was asked for a run ago
+                const int t0 = (run - 1) * SCAN_T;
+                const float* from = s_s[(run - 1) & 1];
 #pragma unroll
-        for (int j = 0; j < SCAN_N; ++j) {
-            const int t = t0 + tt + j * (THREADS / SCAN_CH);
-            if (t < n && live) store_f(out, (size_t)(first + t) * width + c, s_s[threadIdx.x + j * THREADS] * gelu_tanh_f(y_now[j] + yb));
+                for (int j = 0; j < SCAN_N; ++j) {
+                    const int t = t0 + tt + j * SCAN_STEP;
+                    if (t < n && live) store_f(out, (size_t)(first + t) * width + c, from[(tt + j * SCAN_STEP) * SCAN_CH + ch] * gelu_tanh_f(y_r[j] + yb));
+                }
+            }
+            if (run < runs) {
+#pragma unroll
+                for (int j = 0; j < SCAN_N; ++j) {
+                    const int t = run * SCAN_T + tt + j * SCAN_STEP;
+                    if (t < n) y_r[j] = proj[(size_t)(first + t) * stride + y_at + c];
+                }
+                store(in_s[(run + 1) & 1]);
+                fetch((run + 2) * SCAN_T);
+            }
         }
     }
     if (walks && live) *s_at = S;
@@ -310,7 +375,7 @@ scan_kernel(const float2* __restrict__ terms, const float* __restrict__ proj, in
 #define STEP_KC 256
 #define STEP_PITCH (STEP_KC + 8)
 
-template <typename TO>
+template <typename TO, int TAPS>
 __global__ void __launch_bounds__(THREADS)
 step_kernel(Filter f, int y_at, const float* __restrict__ y_bias, const bf16_t* __restrict__ w, const float* __restrict__ r_bias,
             const float* __restrict__ i_bias, const float* __restrict__ decay, float* __restrict__ state, size_t state_stride,
@@ -318,11 +383,16 @@ step_kernel(Filter f, int y_at, const float* __restrict__ y_bias, const bf16_t* 
             TO* __restrict__ out, int tokens, int size, int col_tiles) {
     __shared__ __attribute__((aligned(16))) bf16_t a_s[3][STEP_ROWS * STEP_PITCH];
     __shared__ float red[4][STEP_ROWS * STEP_COLS];
+    __shared__ int p_s[STEP_ROWS], slot_s[STEP_ROWS];
     const int block = blockIdx.x / col_tiles, c0 = (blockIdx.x - block * col_tiles) * STEP_COLS;
     const int t0 = blockIdx.y * STEP_ROWS, rows = min(STEP_ROWS, tokens - t0);
     const int tid = threadIdx.x, wave = tid / KIPP_WAVE, lane = tid & (KIPP_WAVE - 1), l16 = lane & 15, h = lane >> 4;
     const int gate = wave & 1, half = wave >> 1;
     const bf16_t* w_row = w + ((size_t)(block * 2 + gate) * size + min(c0 + l16, size - 1)) * size + 8 * h;
+    if (tid < rows) {
+        p_s[tid] = positions[t0 + tid];
+        slot_s[tid] = slots[seq_of_token[t0 + tid]];
+    }
     f32x4 acc = (f32x4){0.0f, 0.0f, 0.0f, 0.0f};
     for (int k0 = 0; k0 < size; k0 += STEP_KC) {
         Frag b[STEP_KC / 64];       // the weights are asked for first
@@ -331,23 +401,18 @@ step_kernel(Filter f, int y_at, const float* __restrict__ y_bias, const bf16_t* 
             const int k = k0 + 32 * (2 * s + half);
             b[s].u = k + 8 * h < size ? *(const u32x4*)(w_row + k) : (u32x4){0u, 0u, 0u, 0u};
         }
-        __syncthreads();            // the numbers before have been multiplied
-        {
-            const int c = block * size + k0 + tid;
-            const bool there = k0 + tid < size;
-#pragma unroll 4
-            for (int r = 0; r < STEP_ROWS; ++r) {
-                float v = 0.0f;
-                if (there && r < rows) {
-                    const int t = t0 + r;
-                    v = filter_at(f, t, t, positions[t], state + (size_t)slots[seq_of_token[t]] * state_stride + f.width, c);
-                }
-                bf16_t hi, mid, lo;
-                split3(v, hi, mid, lo);
-                a_s[0][r * STEP_PITCH + tid] = hi;
-                a_s[1][r * STEP_PITCH + tid] = mid;
-                a_s[2][r * STEP_PITCH + tid] = lo;
-            }
+        const bool there = k0 + tid < size;
+        const Channel<TAPS> channel(f, block * size + (there ? k0 + tid : 0));
+        __syncthreads();            // the numbers before have been multiplied (and the rows' places are known)
+#pragma unroll(TAPS > 0 ? 8 : 1)
+        for (int r = 0; r < STEP_ROWS; ++r) {
+            float v = 0.0f;
+            if (there && r < rows) v = channel.at(f, t0 + r, t0 + r, p_s[r], state + (size_t)slot_s[r] * state_stride + f.width);
+            __bf16 hi, mid, lo;
+            split3(v, hi, mid, lo);
+            a_s[0][r * STEP_PITCH + tid] = __builtin_bit_cast(bf16_t, hi);
+            a_s[1][r * STEP_PITCH + tid] = __builtin_bit_cast(bf16_t, mid);
+            a_s[2][r * STEP_PITCH + tid] = __builtin_bit_cast(bf16_t, lo);
         }
         __syncthreads();
 #pragma unroll
@@ -368,10 +433,10 @@ step_kernel(Filter f, int y_at, const float* __restrict__ y_bias, const bf16_t* 
     __syncthreads();
     const int r = tid / STEP_COLS, col = c0 + (tid & (STEP_COLS - 1));
     if (r >= rows || col >= size) return;
-    const int t = t0 + r, c = block * size + col, p = positions[t];
-    float* slot = state + (size_t)slots[seq_of_token[t]] * state_stride;
+    const int t = t0 + r, c = block * size + col, p = p_s[r];
+    float* slot = state + (size_t)slot_s[r] * state_stride;
     float* ring = slot + f.width;
-    const float u = filter_at(f, t, t, p, ring, c);
+    const float u = Channel<TAPS>(f, c).at(f, t, t, p, ring);
     const float2 v = recurrence_terms(red[0][tid] + red[2][tid] + r_bias[c], red[1][tid] + red[3][tid] + i_bias[c], decay[c], u);
     const float S = fmaf(v.x, slot[c], v.y);
     slot[c] = S;
@@ -391,8 +456,13 @@ int kipp_recurrence_filter(const float* proj, int stride, int x_at, const float*
     if (taps < 1 || taps > MAX_TAPS || width <= 0 || stride < x_at + width || state_stride < (size_t)(1 + taps) * width) return -1;
     const Filter f = {proj, stride, x_at, x_bias, conv_w, conv_b, taps, width};
     const int cols = (width + THREADS - 1) / THREADS;
-    hipLaunchKernelGGL(filter_kernel, dim3(tokens, cols), dim3(THREADS), 0, stream, f, (const float*)state, state_stride, positions,
-                       seq_of_token, q_start, slots, u);
+    dim3 grid((tokens + FILTER_TOKENS - 1) / FILTER_TOKENS, cols);
+    if (taps == 4)
+        hipLaunchKernelGGL(filter_kernel<4>, grid, dim3(THREADS), 0, stream, f, (const float*)state, state_stride, positions, seq_of_token,
+                           q_start, slots, u, tokens);
+    else
+        hipLaunchKernelGGL(filter_kernel<0>, grid, dim3(THREADS), 0, stream, f, (const float*)state, state_stride, positions, seq_of_token,
+                           q_start, slots, u, tokens);
     hipLaunchKernelGGL(keep_kernel, dim3(cols, entries), dim3(THREADS), 0, stream, f, state, state_stride, positions, q_start, q_len, slots);
     return KIPP_LAUNCH_CHECK();
 }
@@ -450,14 +520,19 @@ int kipp_recurrence_step(const float* proj, int stride, int y_at, int x_at, cons
     const int size = width / blocks, col_tiles = (size + STEP_COLS - 1) / STEP_COLS;
     const Filter f = {proj, stride, x_at, x_bias, conv_w, conv_b, taps, width};
     dim3 grid(blocks * col_tiles, (tokens + STEP_ROWS - 1) / STEP_ROWS);
-    if (out_dtype == KIPP_F32)
-        hipLaunchKernelGGL(step_kernel<float>, grid, dim3(THREADS), 0, stream, f, y_at, y_bias, (const bf16_t*)w, r_bias, i_bias, decay,
-                           state, state_stride, positions, seq_of_token, slots, (float*)out, tokens, size, col_tiles);
-    else if (out_dtype == KIPP_BF16)
-        hipLaunchKernelGGL(step_kernel<bf16_t>, grid, dim3(THREADS), 0, stream, f, y_at, y_bias, (const bf16_t*)w, r_bias, i_bias, decay,
-                           state, state_stride, positions, seq_of_token, slots, (bf16_t*)out, tokens, size, col_tiles);
-    else
+#define KIPP_RS(TO, TAPS)                                                                                                          \
+    hipLaunchKernelGGL((step_kernel<TO, TAPS>), grid, dim3(THREADS), 0, stream, f, y_at, y_bias, (const bf16_t*)w, r_bias, i_bias, decay, \
+                       state, state_stride, positions, seq_of_token, slots, (TO*)out, tokens, size, col_tiles)
+    if (out_dtype == KIPP_F32) {
+        if (taps == 4) KIPP_RS(float, 4);
+        else KIPP_RS(float, 0);
+    } else if (out_dtype == KIPP_BF16) {
+        if (taps == 4) KIPP_RS(bf16_t, 4);
+        else KIPP_RS(bf16_t, 0);
+    } else {
         return -2;
+    }
+#undef KIPP_RS
     return KIPP_LAUNCH_CHECK();
 }
 

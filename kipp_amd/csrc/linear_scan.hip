@@ -331,32 +331,43 @@ extern "C" int kipp_gated_scan(const float* prep, int stride, float* state, size
 
 #define SSD_MAX_HEADS 1024
 
-// One workgroup a token.  proj: [z: inner | x: inner | B: groups n | C: groups n | dt: heads] (inner = heads p); the
-// channels x | B | C pass a causal filter (conv_w [channels][taps] with conv_b [channels], the slot's kept inputs ahead of a
-// portion; kept [taps - 1][channels] at `kept_at` floats into the slot) and silu.  prep as `kipp_gated_scan` reads it.
+// A thread a channel, for TOKENS tokens in a row.  proj: [z: inner | x: inner | B: groups n | C: groups n | dt: heads] (inner =
+// heads p); the channels x | B | C pass a causal filter (conv_w [channels][taps] with conv_b [channels], the slot's kept inputs
+// ahead of a portion; kept [taps - 1][channels] at `kept_at` floats into the slot) and silu.  prep as `kipp_gated_scan` reads it.
+template <int TOKENS>
 __global__ void __launch_bounds__(SCAN_THREADS)
 ssd_prepare_kernel(const float* __restrict__ proj, int stride, const float* __restrict__ conv_w, const float* __restrict__ conv_b, int taps,
                    const float* __restrict__ a_log, const float* __restrict__ dt_bias, const float* __restrict__ state,
                    size_t state_stride, size_t kept_at, const int32_t* __restrict__ seq_of_token,
                    const int32_t* __restrict__ q_start, const int32_t* __restrict__ slots, float* __restrict__ prep,
-                   int prep_stride, int heads, int groups, int n, int p) {
-    __shared__ float dt_s[SSD_MAX_HEADS];
-    const int t = blockIdx.x;
-    const int entry = seq_of_token[t];
-    const int first = q_start[entry];
+                   int prep_stride, int tokens, int heads, int groups, int n, int p) {
+    const int t0 = blockIdx.x * TOKENS;
     const int inner = heads * p, gn = groups * n;
     const int channels = inner + 2 * gn;
-    const float* kept = state + (size_t)slots[entry] * state_stride + kept_at;
-    const float* row = proj + (size_t)t * stride;
-    float* dst = prep + (size_t)t * prep_stride;
-    for (int h = threadIdx.x; h < heads; h += SCAN_THREADS) {
-        const float dt = softplus_f(row[2 * inner + 2 * gn + h] + dt_bias[h]);
-        dt_s[h] = dt;
-        dst[2 * gn + 2 * inner + h] = expf(-expf(a_log[h]) * dt);
+    const int c = blockIdx.y * SCAN_THREADS + threadIdx.x;
+    const int dt_at = 2 * inner + 2 * gn;
+    if (blockIdx.y == 0) {
+        for (int i = threadIdx.x; i < TOKENS * heads; i += SCAN_THREADS) {
+            const int t = t0 + i / heads, h = i % heads;
+            if (t < tokens)
+                prep[(size_t)t * prep_stride + 2 * gn + 2 * inner + h] =
+                    expf(-expf(a_log[h]) * softplus_f(proj[(size_t)t * stride + dt_at + h] + dt_bias[h]));
+        }
     }
-    __syncthreads();
-    for (int c = threadIdx.x; c < channels; c += SCAN_THREADS) {
-        float y = conv_b[c];
+    if (c >= channels) return;
+    const float bias = conv_b[c];
+    const int h = c < inner ? c / p : 0;
+    const float dtb = dt_bias[h];
+#pragma unroll
+    for (int i = 0; i < TOKENS; ++i) {
+        const int t = t0 + i;
+        if (t >= tokens) break;
+        const int entry = seq_of_token[t];
+        const int first = q_start[entry];
+        const float* kept = state + (size_t)slots[entry] * state_stride + kept_at;
+        float* dst = prep + (size_t)t * prep_stride;
+        const float z = c < inner ? proj[(size_t)t * stride + dt_at + h] : 0.0f;
+        float y = bias;
         for (int j = 0; j < taps; ++j) {
             const int at = t - (taps - 1) + j;      // the row of the input `taps - 1 - j` tokens back
             const float in = at >= first ? proj[(size_t)at * stride + inner + c] : kept[(size_t)(taps - 1 + (at - first)) * channels + c];
@@ -364,7 +375,7 @@ ssd_prepare_kernel(const float* __restrict__ proj, int stride, const float* __re
         }
         y = silu_f(y);
         if (c < inner) {
-            dst[2 * gn + c] = dt_s[c / p] * y;
+            dst[2 * gn + c] = softplus_f(z + dtb) * y;
             dst[2 * gn + inner + c] = y;
         } else if (c < inner + gn) {
             dst[gn + (c - inner)] = y;          // B: the keys
@@ -383,8 +394,14 @@ extern "C" int kipp_ssd_prepare(const float* proj, int stride, const float* conv
     const int inner = heads * p, channels = inner + 2 * groups * n;
     if (stride < inner + channels + heads || prep_stride < 2 * groups * n + 2 * inner + heads ||
         state_stride < kept_at + (size_t)(taps - 1) * channels) return -1;
-    hipLaunchKernelGGL(ssd_prepare_kernel, dim3(tokens), dim3(SCAN_THREADS), 0, stream, proj, stride, conv_w, conv_b, taps, a_log, dt_bias,
-                       (const float*)state, state_stride, kept_at, seq_of_token, q_start, slots, prep, prep_stride, heads, groups, n, p);
+    const int cols = (channels + SCAN_THREADS - 1) / SCAN_THREADS;
+#define KIPP_SP(TOKENS)                                                                                                               \
+    hipLaunchKernelGGL(ssd_prepare_kernel<TOKENS>, dim3((tokens + TOKENS - 1) / TOKENS, cols), dim3(SCAN_THREADS), 0, stream, proj, stride, \
+                       conv_w, conv_b, taps, a_log, dt_bias, (const float*)state, state_stride, kept_at, seq_of_token, q_start, slots, prep, \
+                       prep_stride, tokens, heads, groups, n, p)
+    if (tokens >= 512) KIPP_SP(4);
+    else KIPP_SP(1);
+#undef KIPP_SP
     if (taps > 1)
         hipLaunchKernelGGL(conv_keep_kernel, dim3((channels + 255) / 256, entries), dim3(256), 0, stream, proj + inner, stride, taps, state,
                            state_stride, kept_at, q_start, q_len, slots, channels);

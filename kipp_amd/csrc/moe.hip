@@ -447,6 +447,40 @@ __global__ void moe_combine_kernel(const float* __restrict__ y, const int32_t* _
     out[i] = acc;
 }
 
+// The same four columns a thread, for widths that are a multiple of 4: blockIdx.x a token, its rows of y asked for eight at a time.
+__global__ void __launch_bounds__(256)
+moe_combine4_kernel(const float* __restrict__ y, const int32_t* __restrict__ place, const float* __restrict__ weight,
+                    const float* __restrict__ shared, int shared_parts, size_t shared_stride, float* __restrict__ out, int width, int top) {
+    const int t = blockIdx.x, c4 = blockIdx.y * 256 + threadIdx.x, w4 = width / 4;
+    if (c4 >= w4) return;
+    float4 acc = make_float4(0.0f, 0.0f, 0.0f, 0.0f);
+    for (int j0 = 0; j0 < top; j0 += 8) {
+        float4 v[8];
+        float by[8];
+#pragma unroll
+        for (int j = 0; j < 8; ++j)
+            if (j0 + j < top) {
+                const size_t pair = (size_t)t * top + j0 + j;
+                by[j] = weight != nullptr ? weight[pair] : 1.0f;
+                v[j] = ((const float4*)y)[(size_t)place[pair] * w4 + c4];
+            }
+#pragma unroll
+        for (int j = 0; j < 8; ++j)
+            if (j0 + j < top) {
+                acc.x = fmaf(by[j], v[j].x, acc.x);
+                acc.y = fmaf(by[j], v[j].y, acc.y);
+                acc.z = fmaf(by[j], v[j].z, acc.z);
+                acc.w = fmaf(by[j], v[j].w, acc.w);
+            }
+    }
+    const size_t at = (size_t)t * w4 + c4;
+    for (int p = 0; p < shared_parts; ++p) {
+        const float4 s = ((const float4*)(shared + p * shared_stride))[at];
+        acc.x += s.x; acc.y += s.y; acc.z += s.z; acc.w += s.w;
+    }
+    ((float4*)out)[at] = acc;
+}
+
 extern "C" int kipp_moe_route(const float* z, int parts, int stride, int32_t* chosen, float* weight, int tokens, int experts, int top,
                               float eps, int32_t* pair_token, int32_t* place_of_pair, int32_t* tiles, int max_tiles, int tile_rows,
                               float* row_weight, hipStream_t stream) {
@@ -534,6 +568,11 @@ extern "C" int kipp_moe_combine(const float* y, const int32_t* place, const floa
                                 float* out, int tokens, int width, int top, hipStream_t stream) {
     if (tokens <= 0) return 0;
     const size_t total = (size_t)tokens * width;
+    if (width % 4 == 0 && (((uintptr_t)y | (uintptr_t)out | (uintptr_t)shared) & 15) == 0) {
+        hipLaunchKernelGGL(moe_combine4_kernel, dim3(tokens, (width / 4 + 255) / 256), dim3(256), 0, stream, y, place, weight, shared,
+                           shared != nullptr ? shared_parts : 0, total, out, width, top);
+        return KIPP_LAUNCH_CHECK();
+    }
     hipLaunchKernelGGL(moe_combine_kernel, dim3((unsigned)((total + 255) / 256)), dim3(256), 0, stream, y, place, weight, shared,
                        shared != nullptr ? shared_parts : 0, total, out, tokens, width, top);
     return KIPP_LAUNCH_CHECK();
