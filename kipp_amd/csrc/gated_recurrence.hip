@@ -268,17 +268,27 @@ gates_mfma_kernel(const float* __restrict__ u, const bf16_t* __restrict__ w, con
     }
 }
 
-// ---- the walk: a workgroup takes (entry, 16 channels).  Its first wave walks a run of 192 tokens out of LDS in order (16
-// lanes, a channel each), while the other three bring the next run from registers into LDS, ask memory for the one after it, and
+// ---- the walk: a workgroup takes (entry, 16 channels).  Its first wave walks a run of 196 tokens out of LDS in order (16
+// lanes, a channel each), while the other seven bring the next run from registers into LDS, ask memory for the one after it, and
 // multiply the run before by the other branch and write it: one barrier a run.
 #define SCAN_CH 16
-#define SCAN_T 192
-#define SCAN_MOVERS (THREADS - KIPP_WAVE)
+#define SCAN_T 196
+#define SCAN_WG 512
+#define SCAN_MOVERS (SCAN_WG - KIPP_WAVE)
 #define SCAN_STEP (SCAN_MOVERS / SCAN_CH)       // tokens the movers take side by side
 #define SCAN_N (SCAN_T / SCAN_STEP)
 
+// Eight tokens of a channel: their terms (read ahead) into the state, one after the other.
+__device__ __forceinline__ void walk8(float& S, const float2 (&v)[8], float* to) {
+    float s[8];
+#pragma unroll
+    for (int e = 0; e < 8; ++e) s[e] = S = fmaf(v[e].x, S, v[e].y);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) to[e * SCAN_CH] = s[e];
+}
+
 template <typename TO>
-__global__ void __launch_bounds__(THREADS)
+__global__ void __launch_bounds__(SCAN_WG)
 scan_kernel(const float2* __restrict__ terms, const float* __restrict__ proj, int stride, int y_at, const float* __restrict__ y_bias,
             float* __restrict__ state, size_t state_stride, const int32_t* __restrict__ q_start, const int32_t* __restrict__ q_len,
             const int32_t* __restrict__ slots, TO* __restrict__ out, int width) {
@@ -300,8 +310,8 @@ scan_kernel(const float2* __restrict__ terms, const float* __restrict__ proj, in
     auto fetch = [&](int t0) {
 #pragma unroll
         for (int j = 0; j < SCAN_N; ++j) {
-            const int t = t0 + tt + j * SCAN_STEP;
-            if (t < n) in_r[j] = terms[(size_t)(first + t) * width + c];
+            const int t = min(t0 + tt + j * SCAN_STEP, n - 1);      // (beyond the entry: its last token, dropped; no branch around a load)
+            in_r[j] = terms[(size_t)(first + t) * width + c];
         }
     };
     auto store = [&](float2* to) {
@@ -321,21 +331,19 @@ scan_kernel(const float2* __restrict__ terms, const float* __restrict__ proj, in
                 const float2* in = in_s[run & 1] + ch;
                 float* to = s_s[run & 1] + ch;
                 const int m = min(SCAN_T, n - run * SCAN_T);
-                float2 v[8], next[8];
+                float2 even[8], odd[8];
+                auto read = [&](float2 (&v)[8], int t) {
+                    const float2* at = in + min(t, SCAN_T - 8) * SCAN_CH;      // (beyond the run: read again and dropped)
 #pragma unroll
-                for (int e = 0; e < 8; ++e) v[e] = in[e * SCAN_CH];
+                    for (int e = 0; e < 8; ++e) v[e] = at[e * SCAN_CH];
+                };
+                read(even, 0);
                 int t = 0;
-                for (; t + 8 <= m; t += 8) {
-                    const int ahead = min(t + 8, SCAN_T - 8);       // (beyond the run: read again and dropped)
-#pragma unroll
-                    for (int e = 0; e < 8; ++e) next[e] = in[(ahead + e) * SCAN_CH];
-#pragma unroll
-                    for (int e = 0; e < 8; ++e) {
-                        S = fmaf(v[e].x, S, v[e].y);
-                        to[(t + e) * SCAN_CH] = S;
-                    }
-#pragma unroll
-                    for (int e = 0; e < 8; ++e) v[e] = next[e];
+                for (; t + 16 <= m; t += 16) {
+                    read(odd, t + 8);
+                    walk8(S, even, to + t * SCAN_CH);
+                    read(even, t + 16);
+                    walk8(S, odd, to + (t + 8) * SCAN_CH);
                 }
                 for (; t < m; ++t) {
                     const float2 one = in[t * SCAN_CH];
@@ -347,17 +355,20 @@ scan_kernel(const float2* __restrict__ terms, const float* __restrict__ proj, in
             if (run > 0) {      // the run before: its other branch was asked for a run ago
                 const int t0 = (run - 1) * SCAN_T;
                 const float* from = s_s[(run - 1) & 1];
+                // every product ahead of the first store: a wait for a load behind a branch around a store waits for the store too
+#pragma unroll
+                for (int j = 0; j < SCAN_N; ++j) y_r[j] = from[(tt + j * SCAN_STEP) * SCAN_CH + ch] * gelu_tanh_f(y_r[j] + yb);
 #pragma unroll
                 for (int j = 0; j < SCAN_N; ++j) {
                     const int t = t0 + tt + j * SCAN_STEP;
-                    if (t < n && live) store_f(out, (size_t)(first + t) * width + c, from[(tt + j * SCAN_STEP) * SCAN_CH + ch] * gelu_tanh_f(y_r[j] + yb));
+                    if (t < n && live) store_f(out, (size_t)(first + t) * width + c, y_r[j]);
                 }
             }
             if (run < runs) {
 #pragma unroll
                 for (int j = 0; j < SCAN_N; ++j) {
-                    const int t = run * SCAN_T + tt + j * SCAN_STEP;
-                    if (t < n) y_r[j] = proj[(size_t)(first + t) * stride + y_at + c];
+                    const int t = min(run * SCAN_T + tt + j * SCAN_STEP, n - 1);
+                    y_r[j] = proj[(size_t)(first + t) * stride + y_at + c];
                 }
                 store(in_s[(run + 1) & 1]);
                 fetch((run + 2) * SCAN_T);
@@ -499,10 +510,10 @@ int kipp_recurrence_scan(const float* terms, const float* proj, int stride, int 
     if (width <= 0 || stride < y_at + width || state_stride < (size_t)width) return -1;
     dim3 grid((width + SCAN_CH - 1) / SCAN_CH, entries);
     if (out_dtype == KIPP_F32)
-        hipLaunchKernelGGL(scan_kernel<float>, grid, dim3(THREADS), 0, stream, (const float2*)terms, proj, stride, y_at, y_bias, state,
+        hipLaunchKernelGGL(scan_kernel<float>, grid, dim3(SCAN_WG), 0, stream, (const float2*)terms, proj, stride, y_at, y_bias, state,
                            state_stride, q_start, q_len, slots, (float*)out, width);
     else if (out_dtype == KIPP_BF16)
-        hipLaunchKernelGGL(scan_kernel<bf16_t>, grid, dim3(THREADS), 0, stream, (const float2*)terms, proj, stride, y_at, y_bias, state,
+        hipLaunchKernelGGL(scan_kernel<bf16_t>, grid, dim3(SCAN_WG), 0, stream, (const float2*)terms, proj, stride, y_at, y_bias, state,
                            state_stride, q_start, q_len, slots, (bf16_t*)out, width);
     else
         return -2;
