@@ -355,7 +355,7 @@ def bipazen_config(qwen: dict, layers: int, kind: str) -> dict:
     that every mechanism's kernels stand beside their like alone: "mamba2" (width / 64 heads of 64 with a state of 128 and a
     filter of 4 taps: Zivazen's state space layer), "rglru" (as wide as the model, in blocks of 256 channels, 4 taps), "latent"
     (16 heads over a cached row of 192 + 64 numbers, every key seen: Rerizen's latent without its window), or "mixed" (mamba2,
-    rglru, rglru, latent in turn, the second time round with the first round's weights).  Every layer has the routed
+    rglru, rglru, latent in turn, a layer beyond the fourth with the weights of the one four before it).  Every layer has the routed
     feed-forward: 32 gated experts of a quarter of the dense inner size, 4 a token, so that a token multiplies as much as in the
     dense layer."""
     width, ff = qwen["hidden_size"], qwen["intermediate_size"]
