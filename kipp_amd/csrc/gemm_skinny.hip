@@ -63,7 +63,6 @@ struct RowScale {               // sumsq == nullptr: none
 struct AddNorm {                // residual == nullptr: none
     float* residual;            // [M, N], updated in place
     const float* norm_w;        // [N]
-    const float* delta_scale;   // [N]: the product's columns times these on their way into the sum (or null)
     bf16_t* rows_out;           // [M, N] = bfloat16(residual * norm_w)
     float* sumsq_out;           // [M, stride]: ceil(N / 16) sums a row, stride as in RowScale
     int stride;
@@ -77,10 +76,11 @@ __device__ __forceinline__ size_t rows_at(int row, int col, int width, int rows,
 
 #define SCALE_LOADS 10          // 16-byte loads of partial sums a lane has in flight: 160 sums of a row, what 2,560 columns give
 
-template <int MT, bool SWIGLU, int KW, int DEPTH, bool TILED>
-__global__ void __launch_bounds__(THREADS) gemm_skinny_kernel(
+// SCALED: the product's columns times delta_scales [N] on their way into the residual.
+template <int MT, bool SWIGLU, int KW, int DEPTH, bool TILED, bool SCALED>
+__device__ __forceinline__ void skinny_product(
     const bf16_t* __restrict__ X, const bf16_t* __restrict__ W, float* Y, bf16_t* __restrict__ act,
-    int M, int N, int K, RowScale rs, AddNorm an, int x_major, int act_major) {
+    int M, int N, int K, RowScale rs, AddNorm an, int x_major, int act_major, const float* __restrict__ delta_scales) {
     constexpr bool PAIRS = SWIGLU && TILED;          // gate and up rows share a tile
     constexpr int NT = SWIGLU && !TILED ? 2 : 1;
     constexpr int TW = WAVES / KW;                   // row tiles of a workgroup
@@ -137,14 +137,14 @@ __global__ void __launch_bounds__(THREADS) gemm_skinny_kernel(
 
     // what the residual end adds to, asked for first as well (nobody writes these elements before that end does)
     const bool wide = (N & 3) == 0;                  // a lane's four columns are 16 aligned bytes
-    float res[MT][4], norm_w[4], delta_scale[4] = {1.0f, 1.0f, 1.0f, 1.0f};
+    float res[MT][4], norm_w[4], delta_scale[4];
     if (!SWIGLU && an.residual != nullptr && slice == 0) {       // the wave that will hold the tile's sums
         const int col = min(n0 + 4 * h, wide ? N - 4 : N - 1);
         if (wide) {
             const float4 w4 = *(const float4*)(an.norm_w + col);
             norm_w[0] = w4.x, norm_w[1] = w4.y, norm_w[2] = w4.z, norm_w[3] = w4.w;
-            if (an.delta_scale != nullptr) {
-                const float4 s4 = *(const float4*)(an.delta_scale + col);
+            if (SCALED) {
+                const float4 s4 = *(const float4*)(delta_scales + col);
                 delta_scale[0] = s4.x, delta_scale[1] = s4.y, delta_scale[2] = s4.z, delta_scale[3] = s4.w;
             }
 #pragma unroll
@@ -157,7 +157,7 @@ __global__ void __launch_bounds__(THREADS) gemm_skinny_kernel(
             for (int v = 0; v < 4; ++v) {
                 const int c = min(n0 + 4 * h + v, N - 1);
                 norm_w[v] = an.norm_w[c];
-                if (an.delta_scale != nullptr) delta_scale[v] = an.delta_scale[c];
+                if (SCALED) delta_scale[v] = delta_scales[c];
 #pragma unroll
                 for (int mt = 0; mt < MT; ++mt) res[mt][v] = an.residual[(size_t)min(16 * mt + l16, M - 1) * N + c];
             }
@@ -308,7 +308,7 @@ __global__ void __launch_bounds__(THREADS) gemm_skinny_kernel(
             float x[4], ss = 0.0f;
 #pragma unroll
             for (int v = 0; v < 4; ++v) {
-                x[v] = fmaf(delta_scale[v], sum[0][mt][v], res[mt][v]);       // (times one: the plain sum's bits)
+                x[v] = SCALED ? fmaf(delta_scale[v], sum[0][mt][v], res[mt][v]) : res[mt][v] + sum[0][mt][v];
                 if (token < M && n + v < N) ss = fmaf(x[v], x[v], ss);
             }
             if (token < M && wide && n + 3 < N) {
@@ -369,9 +369,24 @@ __global__ void __launch_bounds__(THREADS) gemm_skinny_kernel(
     }
 }
 
+// Two kernels of it: the one with the columns' factors takes an argument more, and the other keeps its argument list as it was.
+template <int MT, bool SWIGLU, int KW, int DEPTH, bool TILED>
+__global__ void __launch_bounds__(THREADS) gemm_skinny_kernel(
+    const bf16_t* __restrict__ X, const bf16_t* __restrict__ W, float* Y, bf16_t* __restrict__ act,
+    int M, int N, int K, RowScale rs, AddNorm an, int x_major, int act_major) {
+    skinny_product<MT, SWIGLU, KW, DEPTH, TILED, false>(X, W, Y, act, M, N, K, rs, an, x_major, act_major, nullptr);
+}
+
+template <int MT, bool SWIGLU, int KW, int DEPTH, bool TILED>
+__global__ void __launch_bounds__(THREADS) gemm_skinny_scaled_kernel(
+    const bf16_t* __restrict__ X, const bf16_t* __restrict__ W, float* Y, bf16_t* __restrict__ act,
+    int M, int N, int K, RowScale rs, AddNorm an, int x_major, int act_major, const float* __restrict__ delta_scales) {
+    skinny_product<MT, SWIGLU, KW, DEPTH, TILED, true>(X, W, Y, act, M, N, K, rs, an, x_major, act_major, delta_scales);
+}
+
 template <bool SWIGLU, int KW, bool TILED>
 static int launch_kw(const bf16_t* X, const bf16_t* W, float* Y, bf16_t* act, int M, int N, int K, int parts,
-                     RowScale rs, AddNorm an, int x_major, int act_major, hipStream_t stream) {
+                     RowScale rs, AddNorm an, int x_major, int act_major, const float* delta_scale, hipStream_t stream) {
     const int inner = SWIGLU ? N / 2 : N;
     const int tiles = SWIGLU && TILED ? (inner + 7) / 8 : (inner + 15) / 16;
     constexpr int TW = WAVES / KW;
@@ -382,9 +397,19 @@ static int launch_kw(const bf16_t* X, const bf16_t* W, float* Y, bf16_t* act, in
 #define KIPP_SK(MT, D) \
     hipLaunchKernelGGL((gemm_skinny_kernel<MT, SWIGLU, KW, D, TILED>), grid, block, 0, stream, X, W, Y, act, M, N, K, rs, an, x_major, \
                        act_major)
+#define KIPP_SKS(MT, D) \
+    hipLaunchKernelGGL((gemm_skinny_scaled_kernel<MT, SWIGLU, KW, D, TILED>), grid, block, 0, stream, X, W, Y, act, M, N, K, rs, an, x_major, \
+                       act_major, delta_scale)
     switch (mt) {
         case 1:
             // fewer workgroups than compute units: what is in flight is what the busy ones ask for, so they ask for twice as much
+            if constexpr (!SWIGLU) {
+                if (an.residual != nullptr && delta_scale != nullptr) {
+                    if (grid.x * grid.y < 256 && K / 32 / 16 >= KW) KIPP_SKS(1, 16);
+                    else KIPP_SKS(1, 8);
+                    break;
+                }
+            }
             if (grid.x * grid.y < 256 && K / 32 / 16 >= KW) KIPP_SK(1, 16);
             else KIPP_SK(1, 8);
             break;
@@ -394,19 +419,20 @@ static int launch_kw(const bf16_t* X, const bf16_t* W, float* Y, bf16_t* act, in
         default: return -1;
     }
 #undef KIPP_SK
+#undef KIPP_SKS
     return KIPP_LAUNCH_CHECK();
 }
 
 template <bool SWIGLU>
 static int launch(const bf16_t* X, const bf16_t* W, float* Y, bf16_t* act, int M, int N, int K, int parts, int kw,
-                  int tiled, RowScale rs, AddNorm an, int x_major, int act_major, hipStream_t stream) {
+                  int tiled, RowScale rs, AddNorm an, int x_major, int act_major, const float* delta_scale, hipStream_t stream) {
     if (tiled && (K & 31)) return -1;
     if (x_major && (K & 31)) return -1;              // whole runs of 32 columns only
     if (an.residual != nullptr && an.steps_major && (N & 31)) return -1;
     if (act_major && ((N / 2) & 31)) return -1;
 #define KIPP_KW(KW)                                                                          \
-    return tiled ? launch_kw<SWIGLU, KW, true>(X, W, Y, act, M, N, K, parts, rs, an, x_major, act_major, stream)         \
-                 : launch_kw<SWIGLU, KW, false>(X, W, Y, act, M, N, K, parts, rs, an, x_major, act_major, stream)
+    return tiled ? launch_kw<SWIGLU, KW, true>(X, W, Y, act, M, N, K, parts, rs, an, x_major, act_major, delta_scale, stream)         \
+                 : launch_kw<SWIGLU, KW, false>(X, W, Y, act, M, N, K, parts, rs, an, x_major, act_major, delta_scale, stream)
     switch (kw) {
         case 1: KIPP_KW(1);
         case 2: KIPP_KW(2);
@@ -485,9 +511,9 @@ int kipp_gemm_skinny_scaled(const void* X, const void* W, float* Y, int M, int N
     if (residual != nullptr && (norm_w == nullptr || rows_out == nullptr || sumsq_out == nullptr || M > 16)) return -1;
     int kw, parts;
     plan((N + 15) / 16, K, residual != nullptr ? 1 : max_parts, &kw, &parts);
-    AddNorm an = {residual, norm_w, delta_scale, (bf16_t*)rows_out, sumsq_out, sumsq_stride((N + 15) / 16), rows_out_steps_major};
+    AddNorm an = {residual, norm_w, (bf16_t*)rows_out, sumsq_out, sumsq_stride((N + 15) / 16), rows_out_steps_major};
     return launch<false>((const bf16_t*)X, (const bf16_t*)W, Y, nullptr, M, N, K, parts, kw, tiled,
-                         row_scale_of(sumsq, sumsq_parts, K, eps), an, x_steps_major, 0, stream);
+                         row_scale_of(sumsq, sumsq_parts, K, eps), an, x_steps_major, 0, delta_scale, stream);
 }
 
 int kipp_gemm_skinny(const void* X, const void* W, float* Y, int M, int N, int K, int max_parts, int tiled,
@@ -508,9 +534,9 @@ int kipp_gemm_skinny_swiglu(const void* X, const void* W, void* act, int M, int 
     if (sumsq != nullptr && (sumsq_parts <= 0 || M > 16)) return -1;
     int kw, parts;
     plan((two_inner / 2 + 7) / 8, K, 1, &kw, &parts);
-    AddNorm none = {nullptr, nullptr, nullptr, nullptr, nullptr, 4, 0};
+    AddNorm none = {nullptr, nullptr, nullptr, nullptr, 4, 0};
     return launch<true>((const bf16_t*)X, (const bf16_t*)W, nullptr, (bf16_t*)act, M, two_inner, K, 1, kw, tiled,
-                        row_scale_of(sumsq, sumsq_parts, K, eps), none, x_steps_major, act_steps_major, stream);
+                        row_scale_of(sumsq, sumsq_parts, K, eps), none, x_steps_major, act_steps_major, nullptr, stream);
 }
 
 }  // extern "C"
