@@ -12,7 +12,7 @@ import os
 from dataclasses import dataclass
 from typing import Callable, Dict
 
-from .specs import (AttentionSpec, BandScaledRopeSpec, ParallelMixerSpec, SSDSpec, ConfigError, DecayAttentionSpec, EmbeddingSpec, GatedDeltaSpec, GatedMLPSpec,
+from .specs import (AttentionSpec, BandScaledRopeSpec, ParallelMixerSpec, SSDSpec, ConfigError, DecayAttentionSpec, DenseMLPSpec, EmbeddingSpec, GatedDeltaSpec, GatedMLPSpec,
                     GatedRecurrenceSpec, HeadSpec, HyperConnectionSpec, LatentAttentionSpec, LayerNormSpec, LayerRun, LayerScaleSpec, LayerSpec, MLSTMSpec,
                     MixedHeadAttentionSpec, ModelSpec, NoPositionSpec, OnePlusRMSNormSpec, RMSNormSpec, RopeSpec,
                     RoutedMLPSpec, ScaledRopeSpec)
@@ -119,3 +119,8 @@ from . import bipazen as _bipazen  # noqa: E402
 
 register_architecture(_bipazen.ARCHITECTURE, _bipazen.BipazenConfig.from_dict)
 BipazenConfig = _bipazen.BipazenConfig
+
+from . import bavedra as _bavedra  # noqa: E402
+
+register_architecture(_bavedra.ARCHITECTURE, _bavedra.BavedraConfig.from_dict)
+BavedraConfig = _bavedra.BavedraConfig

@@ -174,7 +174,8 @@ class AttentionSpec:
     `out_bias` name: the output projection has a bias of that local name.  `v_mix`: "source": this run's values (before
     any mixing) are what later runs of the same step mix in; "mix": v <- (1 - lambda) v + lambda v_source before it is
     cached, lambda the one number of the tensor `v_mix_name`, v_source the source run's values of the same token (a
-    source declares the tensor too and leaves it unused).
+    source declares the tensor too and leaves it unused).  `keys_as_values`: there is no value projection; a value is its
+    token's key as projected (with its bias, before head norm and rotation).
     """
     hidden_size: int
     num_heads: int
@@ -202,10 +203,14 @@ class AttentionSpec:
     out_bias: Optional[str] = None
     v_mix: Optional[str] = None
     v_mix_name: str = "vmix"
+    keys_as_values: bool = False
 
     def __post_init__(self):
         if self.num_heads <= 0 or self.num_kv_heads <= 0:
             raise ConfigError("attention needs at least one query head and one key/value head")
+        if self.keys_as_values and (self.value_dim != self.head_dim or not self.own_kv or self.v_mix is not None or self.v_norm_eps is not None):
+            raise ConfigError(f"attention: keys that are the values need values as wide as keys (here {self.value_dim} and {self.head_dim}), "
+                              f"keys of the mixer's own, and no value norm or mixing")
         if self.chunk is not None and (self.chunk <= 0 or self.window is not None):
             raise ConfigError("attention chunk must be positive and stands instead of a window")
         if self.v_mix not in (None, "source", "mix"):
@@ -261,7 +266,7 @@ class AttentionSpec:
         """None of the extras: the mixer's first kernels (weighted norm, rotation, fused decode) apply."""
         return not self.bias and self.qk_norm_weight and self.q_temp is None and self.v_head_dim is None and self.own_kv \
             and self.softcap is None and self.head_temp is None and self.v_norm_eps is None \
-            and self.chunk is None and not self.sink and self.v_mix is None
+            and self.chunk is None and not self.sink and self.v_mix is None and not self.keys_as_values
 
 
 @dataclass(frozen=True)
@@ -491,13 +496,20 @@ class GatedRecurrenceSpec:
 @dataclass(frozen=True)
 class ParallelMixerSpec:
     """Two mixers side by side that read the same input: delta = left_scale * left(x) + right_scale * right(x).  At most one
-    of them keeps keys and values in pages and at most one keeps state of fixed size."""
+    of them keeps keys and values in pages and at most one keeps state of fixed size.  `left_norm` and `right_norm` (both or
+    neither): RMS norms of the two results over the model's width, delta = left_scale * N_l(left(x)) + right_scale * N_r(right(x))."""
     left: object
     right: object
     left_scale: float = 1.0
     right_scale: float = 1.0
     prefix: str = ""
     kind: str = "parallel_mixer"
+    left_norm: Optional[RMSNormSpec] = None
+    right_norm: Optional[RMSNormSpec] = None
+
+    def __post_init__(self):
+        if (self.left_norm is None) != (self.right_norm is None):
+            raise ConfigError("two mixers side by side: both results are normed, or neither")
 
 
 @dataclass(frozen=True)
@@ -600,16 +612,37 @@ class GatedMLPSpec:
 
 
 @dataclass(frozen=True)
+class DenseMLPSpec:
+    """down(act(up(x))), without a gate and without biases; `activation` is "relu2" (the square of relu), "relu", "silu", "gelu"
+    (the exact one, with erf) or "gelu_tanh".  `names`: the local tensor names of (up, down)."""
+    hidden_size: int
+    intermediate_size: int
+    activation: str = "relu2"
+    prefix: str = ""
+    kind: str = "dense_mlp"
+    names: Tuple[str, str] = ("up", "down")
+
+    def __post_init__(self):
+        if self.intermediate_size <= 0:
+            raise ConfigError("intermediate_size must be positive")
+        if self.activation not in ("gelu", "gelu_tanh", "silu", "relu", "relu2"):
+            raise ConfigError(f"activation {self.activation!r} unsupported (gelu, gelu_tanh, silu, relu, relu2)")
+
+
+@dataclass(frozen=True)
 class RoutedMLPSpec:
     """A mixture of `experts` small feed-forwards, of which a token uses `top`: W_down_e act(W_up_e x), `activation`
     "gelu" (the exact one, with erf), "gelu_tanh", "silu", "relu" or "relu2".  p = softmax(W_router x) over all experts in float32; the
     `top` largest are chosen (the lower index first among equals) and weigh their experts' results by p / (sum of the
     chosen p + `weight_eps`).  `shared_size` I: one more expert of inner size I (tensors under `shared_prefix`) runs for
     every token and is added (None: none).  Expert e's tensors are `expert_prefix.format(e)` + (up, down).
-    `activation` "relu2" is the square of relu.  `router` "sigmoid": scores s = sigmoid(W_router x); the choice goes by
-    s + the tensor `correction_name` (None: no correction); with `groups` (count, keep) the experts form `count` equal groups
-    of neighbours, a group's score is the sum of its two largest choice scores, and only experts of the `keep` best groups can
-    be chosen; weights are s / (sum of the chosen s + `weight_eps`) * `route_scale`, or, `renormalize` False, s * `route_scale`.
+    `activation` "relu2" is the square of relu.  `router` "sigmoid": scores s = sigmoid(W_router x) in the place of p.  The
+    choice goes by s + the tensor `correction_name` (None: no correction); with `groups` (count, keep) the experts form `count`
+    equal groups of neighbours, a group's score is the sum of its two largest choice scores (`group_score` "top2") or its largest
+    ("top1"), and only experts of the `keep` best groups can be chosen; weights are s / (sum of the chosen s + `weight_eps`) *
+    `route_scale`, or, `renormalize` False, s * `route_scale`.  `identity` I: the router has I outputs more, behind the experts';
+    an expert chosen among those is the identity (its result is x; it has no tensors); they take part in softmax, groups and choice.
+    `shared_gate_name`: the shared expert's result is multiplied by sigmoid(w x), w [1, hidden] the tensor of that name.
     `gate_name`: an expert has a third matrix of that local name and is W_down_e (act(W_gate_e x) * (W_up_e x)) (the shared one
     likewise).  `weigh_input`: a weight multiplies its expert's input, not its result: sum of E_e(weight_e x)."""
     hidden_size: int
@@ -632,22 +665,36 @@ class RoutedMLPSpec:
     renormalize: bool = True
     gate_name: Optional[str] = None
     weigh_input: bool = False
+    group_score: str = "top2"
+    identity: int = 0
+    shared_gate_name: Optional[str] = None
+
+    @property
+    def choices(self) -> int:
+        """Outputs of the router: experts and identity experts."""
+        return self.experts + self.identity
 
     def __post_init__(self):
+        if self.identity < 0 or self.group_score not in ("top1", "top2"):
+            raise ConfigError(f"routed feed-forward: identity experts from 0 on (got {self.identity}), a group's score top1 or top2 (got {self.group_score!r})")
+        if self.identity and self.weigh_input:
+            raise ConfigError("routed feed-forward: identity experts with weights on the input are not implemented")
+        if self.shared_gate_name is not None and self.shared_size is None:
+            raise ConfigError("routed feed-forward: a gate of the shared expert needs a shared expert")
         if self.weigh_input and self.gate_name is None:
             raise ConfigError("routed feed-forward: weights on the input are implemented for experts with a gate")
         if self.router not in ("softmax", "sigmoid"):
             raise ConfigError(f"routed feed-forward: router {self.router!r} is not one of softmax, sigmoid")
-        if self.router == "softmax" and (self.correction_name is not None or self.groups is not None or self.route_scale != 1.0 or not self.renormalize):
-            raise ConfigError("routed feed-forward: a correction, groups, a scale and weights as they are belong to the sigmoid router")
+        if self.router == "softmax" and not self.renormalize:
+            raise ConfigError("routed feed-forward: weights as they are belong to the sigmoid router")
         if self.groups is not None:
             count, keep = self.groups
-            if count <= 0 or self.experts % count or not 0 < keep <= count or self.top > keep * (self.experts // count):
-                raise ConfigError(f"routed feed-forward: groups {self.groups}: equal groups of the {self.experts} experts, of which "
+            if count <= 0 or self.choices % count or not 0 < keep <= count or self.top > keep * (self.choices // count):
+                raise ConfigError(f"routed feed-forward: groups {self.groups}: equal groups of the {self.choices} experts, of which "
                                   f"1 to count stay, with experts enough for the {self.top} a token uses")
-        if not 0 < self.top <= self.experts:
-            raise ConfigError(f"routed feed-forward: top {self.top} must be from 1 to experts {self.experts}")
-        if self.experts > 1024 or self.top > 32:
+        if self.experts <= 0 or not 0 < self.top <= self.choices:
+            raise ConfigError(f"routed feed-forward: top {self.top} must be from 1 to the number of experts, {self.choices}")
+        if self.choices > 1024 or self.top > 32:
             raise ConfigError("routed feed-forward: up to 1,024 experts, up to 32 a token")
         if self.expert_size <= 0 or (self.shared_size is not None and self.shared_size <= 0):
             raise ConfigError("routed feed-forward: inner sizes must be positive")
@@ -660,7 +707,7 @@ class LayerSpec:
     """One block: `block` names the arrangement, `parts` its parts by role.
 
     The "pre_norm" arrangement has the roles mixer_norm, mixer, ffn_norm, ffn
-    and computes x += mixer(mixer_norm(x)); x += ffn(ffn_norm(x)).  The "post_norm"
+    and computes x += mixer(mixer_norm(x)); x += ffn(ffn_norm(x)); "pre_norm_mixer" is its first half alone.  The "post_norm"
     arrangement has the same roles and norms after the sum, the sublayers reading x
     itself: x = mixer_norm(a x + mixer(x)); x = ffn_norm(a x + ffn(x)) with
     a = `residual_scale`; "post_norm_mixer" is its first half alone.  "hyper_pre_norm" keeps

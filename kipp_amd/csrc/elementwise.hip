@@ -405,6 +405,181 @@ __global__ void __launch_bounds__(256) scaled_add_rmsnorm_rows_kernel(float* __r
     }
 }
 
+// Sublayer results that are normed before they are added, and the next norm, in one pass over a row:
+//     x <- x + sum_i scale_i * N_i(sum of the slabs of delta_i);   out = N_next(x)  (out optional)
+// N(u) = u * rsqrt(mean(u^2) + eps) * w, each with an eps and a weight of its own; one or two terms.  Everything is float32.
+struct NormedTerms {
+    const float* delta[2];
+    const float* weight[2];
+    int parts[2];
+    float eps[2], scale[2];
+};
+
+// Two sums over a workgroup at the price of one (scratch: 32 floats).
+__device__ __forceinline__ float2 block_sum2(float a, float b, float* scratch) {
+    const int lane = threadIdx.x & (KIPP_WAVE - 1), wave = threadIdx.x / KIPP_WAVE;
+    const int waves = (blockDim.x + KIPP_WAVE - 1) / KIPP_WAVE;
+    a = wave_sum(a);
+    b = wave_sum(b);
+    __syncthreads();
+    if (lane == 0) {
+        scratch[2 * wave] = a;
+        scratch[2 * wave + 1] = b;
+    }
+    __syncthreads();
+    float2 total = make_float2(0.0f, 0.0f);
+    for (int w = 0; w < waves; ++w) {
+        total.x += scratch[2 * w];
+        total.y += scratch[2 * w + 1];
+    }
+    return total;
+}
+
+// Any width: the row is read again for every step.
+template <int TERMS, typename TO>
+__global__ void __launch_bounds__(256) normed_sum_kernel(float* __restrict__ x, NormedTerms t, const float* __restrict__ next_w, float next_eps,
+                                                         TO* __restrict__ out, int width, size_t part_stride) {
+    __shared__ float scratch[32];
+    const size_t base = (size_t)blockIdx.x * width;
+    auto term = [&](int k, int i) {
+        float d = 0.0f;
+        for (int p = 0; p < t.parts[k]; ++p) d += t.delta[k][p * part_stride + base + i];
+        return d;
+    };
+    float ss[2] = {0.0f, 0.0f};
+    for (int i = threadIdx.x; i < width; i += 256)
+#pragma unroll
+        for (int k = 0; k < TERMS; ++k) {
+            const float d = term(k, i);
+            ss[k] = fmaf(d, d, ss[k]);
+        }
+    const float2 sums = block_sum2(ss[0], ss[1], scratch);
+    float inv[2];
+#pragma unroll
+    for (int k = 0; k < TERMS; ++k) inv[k] = 1.0f / sqrtf((k == 0 ? sums.x : sums.y) / (float)width + t.eps[k]);
+    float next = 0.0f;
+    for (int i = threadIdx.x; i < width; i += 256) {
+        float v = x[base + i];
+#pragma unroll
+        for (int k = 0; k < TERMS; ++k) v = fmaf(t.scale[k], term(k, i) * inv[k] * t.weight[k][i], v);
+        x[base + i] = v;
+        next = fmaf(v, v, next);
+    }
+    if (out == nullptr) return;     // uniform
+    const float s = 1.0f / sqrtf(block_sum(next, scratch) / (float)width + next_eps);
+    for (int i = threadIdx.x; i < width; i += 256) store_f(out, base + i, x[base + i] * s * next_w[i]);
+}
+
+// The same for widths that are a multiple of 4 and at most 4 * THREADS * CH: a row stays in registers.
+template <int TERMS, typename TO, int CH, int THREADS>
+__global__ void __launch_bounds__(THREADS) normed_sum_rows_kernel(float* __restrict__ x, NormedTerms t, const float* __restrict__ next_w,
+                                                                  float next_eps, TO* __restrict__ out, int width, size_t part_stride) {
+    __shared__ float scratch[32];
+    const int n4 = width / 4;
+    const size_t base4 = (size_t)blockIdx.x * n4;
+    const float4 zero = make_float4(0.0f, 0.0f, 0.0f, 0.0f);
+    float4 v[CH], d[TERMS][CH], w[TERMS][CH], nw[CH];
+    // every first load is issued before anything is added
+#pragma unroll
+    for (int c = 0; c < CH; ++c) {
+        const int i = threadIdx.x + c * THREADS;
+        v[c] = nw[c] = zero;
+#pragma unroll
+        for (int k = 0; k < TERMS; ++k) d[k][c] = w[k][c] = zero;
+        if (i < n4) {
+#pragma unroll
+            for (int k = 0; k < TERMS; ++k) {
+                d[k][c] = load4(t.delta[k], base4 + i);
+                w[k][c] = load4(t.weight[k], (size_t)i);
+            }
+            v[c] = load4(x, base4 + i);
+            if (out != nullptr) nw[c] = load4(next_w, (size_t)i);
+        }
+    }
+    float ss[2] = {0.0f, 0.0f};
+#pragma unroll
+    for (int k = 0; k < TERMS; ++k) {
+        for (int p0 = 1; p0 < t.parts[k]; p0 += 4) {        // slabs in order, four asked for at a time
+            float4 more[CH][4];
+#pragma unroll
+            for (int c = 0; c < CH; ++c) {
+                const int i = threadIdx.x + c * THREADS;
+#pragma unroll
+                for (int q = 0; q < 4; ++q) more[c][q] = i < n4 && p0 + q < t.parts[k] ? load4(t.delta[k], (p0 + q) * (part_stride / 4) + base4 + i) : zero;
+            }
+#pragma unroll
+            for (int c = 0; c < CH; ++c)
+#pragma unroll
+                for (int q = 0; q < 4; ++q) {
+                    d[k][c].x += more[c][q].x;
+                    d[k][c].y += more[c][q].y;
+                    d[k][c].z += more[c][q].z;
+                    d[k][c].w += more[c][q].w;
+                }
+        }
+#pragma unroll
+        for (int c = 0; c < CH; ++c) {
+            ss[k] = fmaf(d[k][c].x, d[k][c].x, ss[k]);
+            ss[k] = fmaf(d[k][c].y, d[k][c].y, ss[k]);
+            ss[k] = fmaf(d[k][c].z, d[k][c].z, ss[k]);
+            ss[k] = fmaf(d[k][c].w, d[k][c].w, ss[k]);
+        }
+    }
+    const float2 sums = block_sum2(ss[0], ss[1], scratch);
+    float inv[2];
+#pragma unroll
+    for (int k = 0; k < TERMS; ++k) inv[k] = 1.0f / sqrtf((k == 0 ? sums.x : sums.y) / (float)width + t.eps[k]);
+    float next = 0.0f;
+#pragma unroll
+    for (int c = 0; c < CH; ++c) {
+        const int i = threadIdx.x + c * THREADS;
+#pragma unroll
+        for (int k = 0; k < TERMS; ++k) {
+            v[c].x = fmaf(t.scale[k], d[k][c].x * inv[k] * w[k][c].x, v[c].x);
+            v[c].y = fmaf(t.scale[k], d[k][c].y * inv[k] * w[k][c].y, v[c].y);
+            v[c].z = fmaf(t.scale[k], d[k][c].z * inv[k] * w[k][c].z, v[c].z);
+            v[c].w = fmaf(t.scale[k], d[k][c].w * inv[k] * w[k][c].w, v[c].w);
+        }
+        if (i < n4) store4(x, base4 + i, v[c]);
+        next = fmaf(v[c].x, v[c].x, next);
+        next = fmaf(v[c].y, v[c].y, next);
+        next = fmaf(v[c].z, v[c].z, next);
+        next = fmaf(v[c].w, v[c].w, next);
+    }
+    if (out == nullptr) return;     // uniform
+    const float s = 1.0f / sqrtf(block_sum(next, scratch) / (float)width + next_eps);
+#pragma unroll
+    for (int c = 0; c < CH; ++c) {
+        const int i = threadIdx.x + c * THREADS;
+        if (i < n4)
+            store4(out, base4 + i, make_float4(v[c].x * s * nw[c].x, v[c].y * s * nw[c].y, v[c].z * s * nw[c].z, v[c].w * s * nw[c].w));
+    }
+}
+
+template <int TERMS, typename TO>
+static void launch_normed_sum(float* x, const NormedTerms& t, const float* next_w, float next_eps, TO* out, int rows, int width,
+                              hipStream_t stream) {
+    const size_t stride = (size_t)rows * width;
+    const int n4 = width / 4;
+#define KIPP_NS(CH, THREADS) hipLaunchKernelGGL((normed_sum_rows_kernel<TERMS, TO, CH, THREADS>), dim3(rows), dim3(THREADS), 0, stream, x, t, next_w, next_eps, out, width, stride)
+    // (workgroups of one size for a width under float32, whatever the rows: a row has the same bits in every batch)
+    if ((width & 3) != 0 || n4 > 2048) {
+        hipLaunchKernelGGL((normed_sum_kernel<TERMS, TO>), dim3(rows), dim3(256), 0, stream, x, t, next_w, next_eps, out, width, stride);
+    } else if (n4 <= 256) {
+        KIPP_NS(1, 256);
+    } else if (sizeof(TO) == 2 && rows <= 256) {
+        if (n4 <= 512) KIPP_NS(1, 512);
+        else if (n4 <= 1024) KIPP_NS(1, 1024);
+        else KIPP_NS(2, 1024);
+    } else {
+        if (n4 <= 512) KIPP_NS(2, 256);
+        else if (n4 <= 768) KIPP_NS(3, 256);
+        else if (n4 <= 1024) KIPP_NS(2, 512);
+        else KIPP_NS(4, 512);
+    }
+#undef KIPP_NS
+}
+
 template <typename TD, typename TO, bool SCALED = false>
 static void launch_rmsnorm(float* x, const void* delta, const float* weight, void* out, int rows, int width, float eps,
                            int parts, hipStream_t stream, const float* dscale = nullptr) {
@@ -537,6 +712,26 @@ int kipp_rmsnorm_scaled_delta(float* x, const float* delta, int parts, const flo
     if (delta == nullptr || dscale == nullptr || parts <= 0) return -1;
     if (out_dtype == KIPP_BF16) launch_rmsnorm<float, bf16_t, true>(x, delta, weight, out, rows, width, eps, parts, stream, dscale);
     else launch_rmsnorm<float, float, true>(x, delta, weight, out, rows, width, eps, parts, stream, dscale);
+    return KIPP_LAUNCH_CHECK();
+}
+
+// x [rows, width] += sum over the terms (one, or two with delta2) of scale * N(delta); out (or null) = N_next(x).
+int kipp_normed_sum_step(float* x, const float* delta1, int parts1, const float* w1, float eps1, float scale1, const float* delta2, int parts2,
+                         const float* w2, float eps2, float scale2, const float* next_w, float next_eps, void* out, int out_dtype, int rows,
+                         int width, hipStream_t stream) {
+    if (rows <= 0) return 0;
+    if (width <= 0 || delta1 == nullptr || w1 == nullptr || parts1 <= 0) return -1;
+    if (delta2 != nullptr && (w2 == nullptr || parts2 <= 0)) return -1;
+    if (out != nullptr && next_w == nullptr) return -1;
+    const NormedTerms t = {{delta1, delta2}, {w1, w2}, {parts1, parts2}, {eps1, eps2}, {scale1, scale2}};
+    const bool half = out != nullptr && out_dtype == KIPP_BF16;
+    if (delta2 != nullptr) {
+        if (half) launch_normed_sum<2, bf16_t>(x, t, next_w, next_eps, (bf16_t*)out, rows, width, stream);
+        else launch_normed_sum<2, float>(x, t, next_w, next_eps, (float*)out, rows, width, stream);
+    } else {
+        if (half) launch_normed_sum<1, bf16_t>(x, t, next_w, next_eps, (bf16_t*)out, rows, width, stream);
+        else launch_normed_sum<1, float>(x, t, next_w, next_eps, (float*)out, rows, width, stream);
+    }
     return KIPP_LAUNCH_CHECK();
 }
 

@@ -17,6 +17,8 @@
 // (W = [gate; up] in paired tiles, act = silu(gate) * up written straight from the sums) needs the whole of K
 // in one workgroup.
 //
+// Another end writes the square of relu of the product as bfloat16 [M, N]; it needs the whole of K in one workgroup too.
+//
 // v_mfma_f32_16x16x32_bf16: A = W tile (lane: row l % 16, k = 8 (l / 16) + j),
 // B = X^T from LDS (lane: token l % 16, same k), D: lane holds features
 // 4 (l / 16) + v of token l % 16.
@@ -39,7 +41,8 @@ union Frag {
 // DEPTH: steps of 32 columns in one chunk.  NTW: 16-row tiles of W a wave streams (every fragment of X
 // read from LDS then serves NTW products, and a workgroup's staging of X serves NTW times the rows).
 // END 1: W is [gate; up] in paired tiles (8 gate rows over the 8 matching up rows), N = 16 tiles' columns, K is not split and
-// act[M, inner] = bfloat16(silu(gate) * up) is written instead of Y.
+// act[M, inner] = bfloat16(silu(gate) * up) is written instead of Y.  END 2: K is not split and act[M, N] =
+// bfloat16(relu(product)^2) is written.
 #define MIN_WAVES 4
 #define MAX_WAVES 8
 
@@ -196,6 +199,23 @@ __global__ void __launch_bounds__(MAX_WAVES * KIPP_WAVE) gemm_rows_kernel(
         for (int mt = 0; mt < MT; ++mt) {
             const int token = 16 * mt + l16;
             if (token >= M) continue;
+            if (END == 2) {
+                bf16_t r[4];
+#pragma unroll
+                for (int v = 0; v < 4; ++v) {
+                    const float z = fmaxf(acc[i][mt][v], 0.0f);
+                    r[v] = f32_to_bf16(z * z);
+                }
+                bf16_t* out = act + (size_t)token * N + n;
+                if (n + 3 < N && (N & 3) == 0) {
+                    *(uint2*)out = make_uint2((uint32_t)r[0] | ((uint32_t)r[1] << 16), (uint32_t)r[2] | ((uint32_t)r[3] << 16));
+                } else {
+#pragma unroll
+                    for (int v = 0; v < 4; ++v)
+                        if (n + v < N) out[v] = r[v];
+                }
+                continue;
+            }
             float* y = Y + ((size_t)part * M + token) * N + n;
             if (n + 3 < N && (N & 3) == 0) {
                 *(float4*)y = make_float4(acc[i][mt][0], acc[i][mt][1], acc[i][mt][2], acc[i][mt][3]);
@@ -264,8 +284,8 @@ static int launch(const void* X, const void* W, float* Y, void* act, int M, int 
         if (tiled)                                                                                                       \
             hipLaunchKernelGGL((gemm_rows_kernel<MT, true, DEPTH, NTW, END>), grid, block, 0, stream, (const bf16_t*)X,  \
                                (const bf16_t*)W, Y, (bf16_t*)act, M, N, K, inner);                                       \
-        else if (END == 0)                                                                                               \
-            hipLaunchKernelGGL((gemm_rows_kernel<MT, false, DEPTH, NTW, 0>), grid, block, 0, stream, (const bf16_t*)X,   \
+        else if (END != 1)                                                                                               \
+            hipLaunchKernelGGL((gemm_rows_kernel<MT, false, DEPTH, NTW, END == 1 ? 0 : END>), grid, block, 0, stream, (const bf16_t*)X,   \
                                (const bf16_t*)W, Y, (bf16_t*)act, M, N, K, inner);                                       \
         else                                                                                                             \
             return -1;                                                                                                   \
@@ -344,6 +364,23 @@ int kipp_gemm_rows_swiglu(const void* X, const void* W, void* act, int M, int tw
     int tw, ntw, parts;
     if (cut_or_plan(M, N, K, 1, cut, &tw, &ntw, &parts) != 0 || parts != 1) return -1;
     return launch<1>(X, W, nullptr, act, M, N, K, inner, tw, ntw, 1, 1, stream);
+}
+
+// Whether the product that ends in the square of relu is taken for this shape (as for SwiGLU's).
+int kipp_gemm_rows_relu2_pays(int M, int N, int K) {
+    if (M <= 0 || M > 64 || N <= 0 || K <= 0 || (K & 7)) return 0;
+    int tw, ntw, parts;
+    const double whole = plan(M, N, K, 1, &tw, &ntw, &parts), split = plan(M, N, K, 12, &tw, &ntw, &parts);
+    return whole <= 1.2 * split;
+}
+
+// act: bfloat16 [M, N] = relu(X . W^T)^2; W [N, K], or its streaming layout (`tiled`, K a multiple of 32).
+int kipp_gemm_rows_relu2(const void* X, const void* W, void* act, int M, int N, int K, int tiled, int cut, hipStream_t stream) {
+    if (M <= 0 || N <= 0) return 0;
+    if (M > MAX_ROWS || K <= 0 || (K & 7) || (tiled && (K & 31))) return -1;
+    int tw, ntw, parts;
+    if (cut_or_plan(M, N, K, 1, cut, &tw, &ntw, &parts) != 0 || parts != 1) return -1;
+    return launch<2>(X, W, nullptr, act, M, N, K, 0, tw, ntw, 1, tiled, stream);
 }
 
 }  // extern "C"

@@ -23,6 +23,9 @@
 // Every request then covers full memory lines, which a compute unit issues at a
 // bounded rate: the same kernel streams a fifth faster than from [N, K] rows.
 //
+// With RELU2 the square of relu of the product is written as bfloat16 [M, N] instead of Y (the product is then not split
+// over workgroups).
+//
 // With SWIGLU the weight is [gate rows; up rows] ([2 I, K]) and the kernel writes
 // silu(gate) * up as bfloat16 [M, I]  (/root/reference/src/kipp.c:2644-2648).
 // From rows, a wave computes a gate tile and the matching up tile together.  In
@@ -77,7 +80,7 @@ __device__ __forceinline__ size_t rows_at(int row, int col, int width, int rows,
 #define SCALE_LOADS 10          // 16-byte loads of partial sums a lane has in flight: 160 sums of a row, what 2,560 columns give
 
 // SCALED: the product's columns times delta_scales [N] on their way into the residual.
-template <int MT, bool SWIGLU, int KW, int DEPTH, bool TILED, bool SCALED>
+template <int MT, bool SWIGLU, int KW, int DEPTH, bool TILED, bool SCALED, bool RELU2 = false>
 __device__ __forceinline__ void skinny_product(
     const bf16_t* __restrict__ X, const bf16_t* __restrict__ W, float* Y, bf16_t* __restrict__ act,
     int M, int N, int K, RowScale rs, AddNorm an, int x_major, int act_major, const float* __restrict__ delta_scales) {
@@ -356,6 +359,20 @@ __device__ __forceinline__ void skinny_product(
                     act[rows_at(token, n + v, inner, M, act_major)] = f32_to_bf16(g / (1.0f + expf(-g)) * up);
                 }
             }
+        } else if (RELU2) {
+            bf16_t r[4];
+#pragma unroll
+            for (int v = 0; v < 4; ++v) {
+                const float z = fmaxf(sum[0][mt][v], 0.0f);
+                r[v] = f32_to_bf16(z * z);
+            }
+            if (n + 3 < N && (N & 3) == 0) {        // four columns of one run of 32
+                *(uint2*)(act + rows_at(token, n, N, M, act_major)) = make_uint2((uint32_t)r[0] | ((uint32_t)r[1] << 16), (uint32_t)r[2] | ((uint32_t)r[3] << 16));
+            } else {
+#pragma unroll
+                for (int v = 0; v < 4; ++v)
+                    if (n + v < N) act[rows_at(token, n + v, N, M, act_major)] = r[v];
+            }
         } else {
             float* y = Y + ((size_t)part * M + token) * N + n;
             if (n + 3 < N && (N & 3) == 0) {
@@ -382,6 +399,36 @@ __global__ void __launch_bounds__(THREADS) gemm_skinny_scaled_kernel(
     const bf16_t* __restrict__ X, const bf16_t* __restrict__ W, float* Y, bf16_t* __restrict__ act,
     int M, int N, int K, RowScale rs, AddNorm an, int x_major, int act_major, const float* __restrict__ delta_scales) {
     skinny_product<MT, SWIGLU, KW, DEPTH, TILED, true>(X, W, Y, act, M, N, K, rs, an, x_major, act_major, delta_scales);
+}
+
+// The square of relu at the end.
+template <int MT, int KW, int DEPTH, bool TILED>
+__global__ void __launch_bounds__(THREADS) gemm_skinny_relu2_kernel(
+    const bf16_t* __restrict__ X, const bf16_t* __restrict__ W, bf16_t* __restrict__ act, int M, int N, int K, RowScale rs, int x_major,
+    int act_major) {
+    const AddNorm none = {nullptr, nullptr, nullptr, nullptr, 4, 0};
+    skinny_product<MT, false, KW, DEPTH, TILED, false, true>(X, W, nullptr, act, M, N, K, rs, none, x_major, act_major, nullptr);
+}
+
+template <int KW, bool TILED>
+static int launch_relu2_kw(const bf16_t* X, const bf16_t* W, bf16_t* act, int M, int N, int K, RowScale rs, int x_major, int act_major,
+                           hipStream_t stream) {
+    constexpr int TW = WAVES / KW;
+    dim3 grid(((N + 15) / 16 + TW - 1) / TW), block(THREADS);
+    if (rs.sumsq != nullptr && M > 16) return -1;
+#define KIPP_SR(MT, D) hipLaunchKernelGGL((gemm_skinny_relu2_kernel<MT, KW, D, TILED>), grid, block, 0, stream, X, W, act, M, N, K, rs, x_major, act_major)
+    switch ((M + 15) / 16) {
+        case 1:
+            if (grid.x < 256 && K / 32 / 16 >= KW) KIPP_SR(1, 16);
+            else KIPP_SR(1, 8);
+            break;
+        case 2: KIPP_SR(2, 8); break;
+        case 3: KIPP_SR(3, 4); break;
+        case 4: KIPP_SR(4, 4); break;
+        default: return -1;
+    }
+#undef KIPP_SR
+    return KIPP_LAUNCH_CHECK();
 }
 
 template <bool SWIGLU, int KW, bool TILED>
@@ -537,6 +584,28 @@ int kipp_gemm_skinny_swiglu(const void* X, const void* W, void* act, int M, int 
     AddNorm none = {nullptr, nullptr, nullptr, nullptr, 4, 0};
     return launch<true>((const bf16_t*)X, (const bf16_t*)W, nullptr, (bf16_t*)act, M, two_inner, K, 1, kw, tiled,
                         row_scale_of(sumsq, sumsq_parts, K, eps), none, x_steps_major, act_steps_major, nullptr, stream);
+}
+
+// act: bfloat16 [M, N] = relu(X . W^T)^2.  W [N, K], or its streaming layout (`tiled`); the rest as above.
+int kipp_gemm_skinny_relu2(const void* X, const void* W, void* act, int M, int N, int K, int tiled, const float* sumsq,
+                           int sumsq_parts, float eps, int x_steps_major, int act_steps_major, hipStream_t stream) {
+    if (M <= 0 || N <= 0) return 0;
+    if (M > 64 || K <= 0 || (K & 7)) return -1;
+    if (sumsq != nullptr && (sumsq_parts <= 0 || M > 16)) return -1;
+    if ((tiled && (K & 31)) || (x_steps_major && (K & 31)) || (act_steps_major && (N & 31))) return -1;
+    int kw, parts;
+    plan((N + 15) / 16, K, 1, &kw, &parts);
+    const RowScale rs = row_scale_of(sumsq, sumsq_parts, K, eps);
+#define KIPP_KR(KW)                                                                                                                     \
+    return tiled ? launch_relu2_kw<KW, true>((const bf16_t*)X, (const bf16_t*)W, (bf16_t*)act, M, N, K, rs, x_steps_major, act_steps_major, stream) \
+                 : launch_relu2_kw<KW, false>((const bf16_t*)X, (const bf16_t*)W, (bf16_t*)act, M, N, K, rs, x_steps_major, act_steps_major, stream)
+    switch (kw) {
+        case 1: KIPP_KR(1);
+        case 2: KIPP_KR(2);
+        case 4: KIPP_KR(4);
+        default: return -1;
+    }
+#undef KIPP_KR
 }
 
 }  // extern "C"

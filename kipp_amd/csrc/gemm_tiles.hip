@@ -24,14 +24,15 @@
 // An output element is summed over K in the same order whatever the tile and the number of waves: cuts
 // with the same parts of K give the same bits.
 //
-// The result leaves through one of three ends:
+// The result leaves through one of four ends:
 //   slabs   float32 [parts, M, N]: K is split over `parts` workgroups (grid.z) where the tiles
 //           alone would leave compute units idle, and the consumer adds the slabs in order
 //           (the residual add, the rotary kernel: no atomics, the same bits every time);
 //   swiglu  W = [gate; up] ([2 I, K]): a wave's columns are gate rows and the up rows that belong
 //           to them, a lane holds both values of an output, and bfloat16(silu(gate) * up)
 //           [M, I] is all that is written (/root/reference/src/kipp.c:2633-2653);
-//   bf16    bfloat16 [M, N].
+//   bf16    bfloat16 [M, N];
+//   relu2   bfloat16 [M, N] = bfloat16(relu(product)^2).
 // The bfloat16 ends pass through LDS so that a lane stores 16 bytes of one row.
 //
 // Tiles are handed to the 8 dies of the GPU in blocks: workgroups that run on one die (every
@@ -55,7 +56,7 @@ union Frag {
 #define LDS_PTR(p) ((__attribute__((address_space(3))) void*)(p))
 #define GLOBAL_PTR(p) ((const __attribute__((address_space(1))) void*)(p))
 
-enum { END_SLABS = 0, END_SWIGLU = 1, END_BF16 = 2 };
+enum { END_SLABS = 0, END_SWIGLU = 1, END_BF16 = 2, END_RELU2 = 3 };
 
 // silu(g) * u with the exponential of the hardware (base 2)
 __device__ __forceinline__ float swiglu_of(float g, float u) {
@@ -353,7 +354,11 @@ __global__ void __launch_bounds__(64 * 2 * WGN, 1) gemm_tiles_kernel(
 #pragma unroll
             for (int v = 0; v < 16; ++v) {
                 const int r = 8 * (v / 4) + 4 * hh + (v % 4);
-                const float value = END == END_SWIGLU ? swiglu_of(acc[i][j][v], acc[i][(j + WN / 2) % WN][v]) : acc[i][j][v];
+                float value = END == END_SWIGLU ? swiglu_of(acc[i][j][v], acc[i][(j + WN / 2) % WN][v]) : acc[i][j][v];
+                if (END == END_RELU2) {
+                    value = fmaxf(value, 0.0f);
+                    value *= value;
+                }
                 stage[r * PITCH + 32 * j + l32] = f32_to_bf16(value);
             }
         // (a wave's lanes run in step: what the wave wrote it can read back without a barrier of the workgroup)
@@ -508,13 +513,13 @@ int kipp_gemm_tiles_parts(int M, int N, int K, int end, int max_parts) {
 }
 
 // Y: float32 [parts, M, N] with parts = kipp_gemm_tiles_parts(...) (end 0), bfloat16 [M, N / 2] = silu(gate) * up for
-// W = [gate; up] (end 1), bfloat16 [M, N] (end 2).  K a multiple of 32.  `force`: 0, or 100 wm + 10 wn + parts (+ 1000: 8 waves, four across; + 2000: the same for whole rounds of tiles, the
+// W = [gate; up] (end 1), bfloat16 [M, N] (end 2), bfloat16 [M, N] = relu(product)^2 (end 3).  K a multiple of 32.  `force`: 0, or 100 wm + 10 wn + parts (+ 1000: 8 waves, four across; + 2000: the same for whole rounds of tiles, the
 // rest of the columns in smaller ones, which + 10000 r chooses) to take that cut whatever the plan says (the runtime's timed choice, tests).
 int kipp_gemm_tiles(const void* X, const void* W, void* Y, int M, int N, int K, int end, int max_parts, int force,
                     hipStream_t stream) {
     if (M <= 0 || N <= 0) return 0;
     if (K <= 0 || (K % BK) || max_parts <= 0) return -1;
-    if (end != END_SLABS && end != END_SWIGLU && end != END_BF16) return -3;
+    if (end != END_SLABS && end != END_SWIGLU && end != END_BF16 && end != END_RELU2) return -3;
     if (end == END_SWIGLU && (N & 1)) return -4;
     // a lane's offset into an operand is 32 bits wide
     if ((unsigned long long)M * K * 2 >= (1ull << 32) || (unsigned long long)N * K * 2 >= (1ull << 32)) return -6;
@@ -533,6 +538,7 @@ int kipp_gemm_tiles(const void* X, const void* W, void* Y, int M, int N, int K, 
         if (cut.parts < 1 || cut.parts > K / BK || (end != END_SLABS && cut.parts != 1)) return -2;
         const int rc = end == END_SLABS ? launch_end<END_SLABS>(X, W, Y, M, N, K, cut, stream)
                        : end == END_SWIGLU ? launch_end<END_SWIGLU>(X, W, Y, M, N, K, cut, stream)
+                       : end == END_RELU2  ? launch_end<END_RELU2>(X, W, Y, M, N, K, cut, stream)
                                            : launch_end<END_BF16>(X, W, Y, M, N, K, cut, stream);
         if (rc != 0) return rc;
     }

@@ -8,8 +8,8 @@
 // one token:
 //     bias    u += bias[column]                               (bias over the q | k | v columns, or none)
 //     norm    u *= rsqrt(mean(u^2) + eps) [* w]               (queries and keys; mode 0 none, 1 plain, 2 weighted)
-//     rotate  queries and keys: number i < r / 2 of a head turns with number i + r / 2 by the token's angle i
-//             (`angles` [tokens][r]: r / 2 cosines, then r / 2 sines; none: no rotation)
+//     rotate  queries and keys: number i < r / 2 of a head turns with number i + r / 2 (`interleaved`: number 2i with number
+//             2i + 1) by the token's angle i (`angles` [tokens][r]: r / 2 cosines, then r / 2 sines; none: no rotation)
 //     factor  queries at position p times 1 + coef * ln(floor((p + 1) / every) + 1)     (every 0: none)
 //     head    queries of head h times q_head_scale[h]                                    (or none)
 //     values  every value head over its root mean square, rsqrt(mean(u^2) + v_norm_eps)  (v_norm_eps < 0: none)
@@ -17,6 +17,8 @@
 //             of the same tokens) the value becomes (1 - lambda) v + lambda v_first, lambda = *v_lambda
 //     write   q to q_out [tokens][n_q d]; the key and value of position p to page table[p / page], slot p % page;
 //             caches [page][kv head][slot][d] and [page][kv head][slot][v_row], v_row >= dv (the rest of a row is zeros)
+// `keys_as_values`: there are no value columns; the wave of a key writes it into the value's row as projected (with its bias) and
+// then, normed and rotated, into the key's.
 // All arithmetic is float32.
 #include "common.h"
 #include <math.h>
@@ -33,12 +35,12 @@ __global__ void head_prepare_kernel(
     const float* __restrict__ k_norm_w, float eps, float temp_coef, int temp_every,
     int n_q, int n_kv, int d, int dv, int page, int write_kv, const float* __restrict__ q_head_scale, float v_norm_eps,
     const float* __restrict__ angles, int rotary_dim, const float* __restrict__ v_first_in, float* __restrict__ v_first_out,
-    const float* __restrict__ v_lambda, int v_row) {
+    const float* __restrict__ v_lambda, int v_row, int interleaved, int keys_as_values) {
     const int wave = threadIdx.x / KIPP_WAVE;
     const int lane = threadIdx.x & (KIPP_WAVE - 1);
     const int t = blockIdx.y;
     const int slot = blockIdx.x * HEADS_PER_BLOCK + wave;
-    const int n_slots = write_kv ? n_q + 2 * n_kv : n_q;
+    const int n_slots = write_kv ? n_q + (keys_as_values ? 1 : 2) * n_kv : n_q;
     if (slot >= n_slots) return;    // no barrier below: a wave is on its own
     const int kind = slot < n_q ? 0 : (slot < n_q + n_kv ? 1 : 2);
     const int head = kind == 0 ? slot : (kind == 1 ? slot - n_q : slot - n_q - n_kv);
@@ -60,6 +62,15 @@ __global__ void head_prepare_kernel(
         vals[c] = v;
         ss = fmaf(v, v, ss);
     }
+    if (kind == 1 && keys_as_values) {
+        const int page_id = block_table[(size_t)seq_of_token[t] * max_blocks + pos / page];
+        TC* dst = v_cache + (((size_t)page_id * n_kv + head) * page + pos % page) * v_row;
+#pragma unroll
+        for (int c = 0; c < MAX_D / KIPP_WAVE; ++c) {
+            const int e = lane + c * KIPP_WAVE;
+            if (e < v_row) store_f(dst, e, e < d ? vals[c] : 0.0f);
+        }
+    }
     if (kind != 2 && norm_mode != 0) {
         ss = wave_sum(ss);
         float scale = 1.0f / sqrtf(ss / (float)d + eps);
@@ -76,7 +87,18 @@ __global__ void head_prepare_kernel(
 #pragma unroll
         for (int c = 0; c < MAX_D / KIPP_WAVE; ++c) vals[c] *= factor;
     }
-    if (kind != 2 && angles != nullptr) {
+    if (kind != 2 && angles != nullptr && interleaved) {
+        // a number's partner is the neighbouring lane's, in the same register
+#pragma unroll
+        for (int c = 0; c < MAX_D / KIPP_WAVE; ++c) {
+            const int e = lane + c * KIPP_WAVE;
+            const float partner = __shfl_xor(vals[c], 1, KIPP_WAVE);
+            if (e < rotary_dim) {
+                const float cs = angles[(size_t)t * rotary_dim + e / 2], sn = angles[(size_t)t * rotary_dim + rotary_dim / 2 + e / 2];
+                vals[c] = (e & 1) ? rotate_hi(partner, vals[c], cs, sn) : rotate_lo(vals[c], partner, cs, sn);
+            }
+        }
+    } else if (kind != 2 && angles != nullptr) {
         // a number's partner lies in another lane (and maybe another register): every lane takes part in every move
         const int half = rotary_dim / 2;
         float turned[MAX_D / KIPP_WAVE];
@@ -148,22 +170,24 @@ extern "C" int kipp_head_prepare_rotated(
     int norm_mode, const float* q_norm_w, const float* k_norm_w, float eps, float temp_coef, int temp_every,
     int n_tokens, int n_q, int n_kv, int d, int dv, int page, int write_kv, const float* q_head_scale, float v_norm_eps,
     const float* angles, int rotary_dim, const float* v_first_in, float* v_first_out, const float* v_lambda, int v_row,
-    hipStream_t stream) {
+    int interleaved, int keys_as_values, hipStream_t stream) {
     if (n_tokens <= 0) return 0;
+    if (keys_as_values && (dv != d || v_first_in != nullptr || v_first_out != nullptr || v_norm_eps >= 0.0f)) return -1;
     if (v_row < dv || v_row > MAX_D) return -1;
     if (angles != nullptr && (rotary_dim <= 0 || rotary_dim % 2 || rotary_dim > d)) return -1;
     if (v_first_in != nullptr && (v_lambda == nullptr || v_first_in == v_first_out)) return -1;
     if (d <= 0 || d > MAX_D || dv <= 0 || dv > MAX_D || n_q <= 0 || n_kv <= 0 || page <= 0) return -1;
-    if (stride < n_q * d + (write_kv ? n_kv * (d + dv) : 0) || norm_mode < 0 || norm_mode > 2 || temp_every < 0) return -1;
+    if (stride < n_q * d + (write_kv ? n_kv * (d + (keys_as_values ? 0 : dv)) : 0) || norm_mode < 0 || norm_mode > 2 || temp_every < 0) return -1;
     if (norm_mode == 2 && (q_norm_w == nullptr || k_norm_w == nullptr)) return -1;
-    const int n_slots = write_kv ? n_q + 2 * n_kv : n_q;
+    const int n_slots = write_kv ? n_q + (keys_as_values ? 1 : 2) * n_kv : n_q;
     dim3 grid((n_slots + HEADS_PER_BLOCK - 1) / HEADS_PER_BLOCK, n_tokens), block(HEADS_PER_BLOCK * KIPP_WAVE);
     const size_t part_stride = (size_t)n_tokens * stride;
 #define KIPP_HP(TO, TC)                                                                                              \
     hipLaunchKernelGGL((head_prepare_kernel<TO, TC>), grid, block, 0, stream, proj, parts, part_stride, stride, bias, \
                        (TO*)q_out, (TC*)k_cache, (TC*)v_cache, positions, seq_of_token, block_table, max_blocks,      \
                        norm_mode, q_norm_w, k_norm_w, eps, temp_coef, temp_every, n_q, n_kv, d, dv, page, write_kv,     \
-                       q_head_scale, v_norm_eps, angles, rotary_dim, v_first_in, v_first_out, v_lambda, v_row)
+                       q_head_scale, v_norm_eps, angles, rotary_dim, v_first_in, v_first_out, v_lambda, v_row, interleaved,     \
+                       keys_as_values)
     if (q_dtype == KIPP_F32 && cache_dtype == KIPP_F32) KIPP_HP(float, float);
     else if (q_dtype == KIPP_BF16 && cache_dtype == KIPP_BF16) KIPP_HP(bf16_t, bf16_t);
     else return -2;
@@ -179,7 +203,8 @@ extern "C" int kipp_head_prepare_scaled(
     hipStream_t stream) {
     return kipp_head_prepare_rotated(proj, parts, stride, bias, q_out, q_dtype, k_cache, v_cache, cache_dtype, positions, seq_of_token,
                                      block_table, max_blocks, norm_mode, q_norm_w, k_norm_w, eps, temp_coef, temp_every, n_tokens, n_q,
-                                     n_kv, d, dv, page, write_kv, q_head_scale, v_norm_eps, nullptr, 0, nullptr, nullptr, nullptr, dv, stream);
+                                     n_kv, d, dv, page, write_kv, q_head_scale, v_norm_eps, nullptr, 0, nullptr, nullptr, nullptr, dv, 0, 0,
+                                     stream);
 }
 
 extern "C" int kipp_head_prepare(

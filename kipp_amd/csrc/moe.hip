@@ -3,11 +3,13 @@
 //
 //     route    p = softmax(z) over all experts (float32); the `top` largest p (the lower index first among equals);
 //              weight = p / (sum of the chosen p + eps)
-//     route (grouped)  s = sigmoid(z); choice scores c = s + correction; experts in equal groups of neighbours, a group's
-//              score the sum of its two largest c; only experts of the `keep` best groups can be chosen; the `top` largest
-//              c among them; weight = s / (sum of the chosen s + eps) * scale, or s * scale (not renormalized)
+//     route (grouped)  s = sigmoid(z), or softmax(z); choice scores c = s + correction; experts in equal groups of neighbours, a
+//              group's score the sum of its two largest c, or its largest; only experts of the `keep` best groups can be chosen; the
+//              `top` largest c among them; weight = s / (sum of the chosen s + eps) * scale, or s * scale (not renormalized)
 //     sort     the (token, choice) pairs in runs of one expert each, cut into tiles of up to 16 (or 128) rows; the list of tiles
-//              is made on the device, so the host never learns the counts and the launches have a fixed shape
+//              is made on the device, so the host never learns the counts and the launches have a fixed shape.  The router may
+//              have more outputs than there are experts with matrices: those behind are identity experts, whose pairs get no
+//              row (place -1)
 //     expert   a tile's rows against its expert's matrix: out[row][n] = act(sum_k W_e[n][k] x[row][k]).  bfloat16 with K a
 //              multiple of 32: on the matrix cores, a workgroup a (tile of up to 128 rows, 128 columns), a wave 32 of the
 //              columns in 8 x 2 fragments of 16 x 16 (two workgroups share a compute unit's registers); steps of 64 numbers of k come from memory 128 bytes a row (eight
@@ -17,7 +19,8 @@
 //     gated expert  the same against an expert's [gate; up] matrix with a weight s a row of x:
 //              out[row][n] = act(s (W_gate x)[n]) * s (W_up x)[n], which is the expert applied to s x; on the matrix cores a wave's
 //              two fragments of 16 columns are the gate's and the up's of the same 16 inner columns
-//     combine  out[t] = sum_j weight[t][j] y[place of (t, j)] (+ the shared expert's result, slabs added in order)
+//     combine  out[t] = sum_j weight[t][j] y[place of (t, j)], or weight[t][j] x[t] for an identity expert (+ the shared expert's
+//              result, slabs added in order, maybe times the sigmoid of a logit of its own)
 #include "common.h"
 #include <math.h>
 
@@ -103,11 +106,12 @@ moe_route_kernel(const float* __restrict__ z, int parts, size_t part_stride, int
     }
 }
 
-// One wave a token: sigmoid scores, a correction for the choice alone, groups of neighbouring experts of which the best stay.
+// One wave a token: sigmoid scores (`softmax`: a softmax over all of them), a correction for the choice alone, groups of
+// neighbouring experts of which the best stay (by the sum of their two largest, or, `by_largest`, by their largest).
 __global__ void __launch_bounds__(ROUTE_WAVES * KIPP_WAVE)
 moe_route_grouped_kernel(const float* __restrict__ z, int parts, size_t part_stride, int stride, const float* __restrict__ correction,
                          int32_t* __restrict__ chosen, float* __restrict__ weight, int tokens, int experts, int top, float eps,
-                         int group_count, int group_keep, float scale, int renormalize) {
+                         int group_count, int group_keep, float scale, int renormalize, int softmax, int by_largest) {
     __shared__ float c_s[ROUTE_WAVES][MAX_EXPERTS];     // choice scores, then -inf for experts of groups that do not stay
     __shared__ float g_s[ROUTE_WAVES][MAX_EXPERTS];     // group scores, -inf once a group is taken
     const int wave = threadIdx.x / KIPP_WAVE, lane = threadIdx.x & (KIPP_WAVE - 1);
@@ -116,6 +120,7 @@ moe_route_grouped_kernel(const float* __restrict__ z, int parts, size_t part_str
     if (!live) t = tokens - 1;      // stay in step with the barriers
     const int size = experts / group_count;
     float s[MAX_EXPERTS / KIPP_WAVE];
+    float m = -INFINITY;
 #pragma unroll
     for (int i = 0; i < MAX_EXPERTS / KIPP_WAVE; ++i) {
         const int e = lane + i * KIPP_WAVE;
@@ -123,9 +128,27 @@ moe_route_grouped_kernel(const float* __restrict__ z, int parts, size_t part_str
         if (e < experts) {
             float v = z[(size_t)t * stride + e];
             for (int q = 1; q < parts; ++q) v += z[q * part_stride + (size_t)t * stride + e];
-            s[i] = 1.0f / (1.0f + expf(-v));
-            c_s[wave][e] = s[i] + (correction != nullptr ? correction[e] : 0.0f);
+            s[i] = softmax ? v : 1.0f / (1.0f + expf(-v));
+            m = fmaxf(m, v);
         }
+    }
+    if (softmax) {
+        m = wave_max(m);
+        float sum = 0.0f;
+#pragma unroll
+        for (int i = 0; i < MAX_EXPERTS / KIPP_WAVE; ++i)
+            if (lane + i * KIPP_WAVE < experts) {
+                s[i] = expf(s[i] - m);
+                sum += s[i];
+            }
+        sum = wave_sum(sum);
+#pragma unroll
+        for (int i = 0; i < MAX_EXPERTS / KIPP_WAVE; ++i) s[i] = s[i] / sum;
+    }
+#pragma unroll
+    for (int i = 0; i < MAX_EXPERTS / KIPP_WAVE; ++i) {
+        const int e = lane + i * KIPP_WAVE;
+        if (e < experts) c_s[wave][e] = s[i] + (correction != nullptr ? correction[e] : 0.0f);
     }
     __syncthreads();
     if (group_keep < group_count) {
@@ -135,7 +158,7 @@ moe_route_grouped_kernel(const float* __restrict__ z, int parts, size_t part_str
                 const float v = c_s[wave][g * size + j];
                 if (v > a) { b = a; a = v; } else if (v > b) { b = v; }
             }
-            g_s[wave][g] = size > 1 ? a + b : a;
+            g_s[wave][g] = size > 1 && !by_largest ? a + b : a;
         }
         __syncthreads();
         for (int round = 0; round < group_keep; ++round) {
@@ -190,7 +213,7 @@ moe_route_grouped_kernel(const float* __restrict__ z, int parts, size_t part_str
 }
 
 // One workgroup sorts all pairs.  tiles: int32 [max_tiles][3] = (expert, first row, rows); rows 0 marks an unused tile.
-// `row_weight` (or null) receives every sorted row's weight.
+// `row_weight` (or null) receives every sorted row's weight.  Choices from `experts` on are identity experts: no row, place -1.
 __global__ void __launch_bounds__(1024)
 moe_sort_kernel(const int32_t* __restrict__ chosen, int pairs, int experts, int top, int32_t* __restrict__ pair_token,
                 int32_t* __restrict__ place_of_pair, int32_t* __restrict__ tiles, int max_tiles, int tile_rows,
@@ -200,7 +223,10 @@ moe_sort_kernel(const int32_t* __restrict__ chosen, int pairs, int experts, int 
     __shared__ int tile_first[MAX_EXPERTS + 1];
     for (int e = threadIdx.x; e < experts; e += blockDim.x) count[e] = 0;
     __syncthreads();
-    for (int p = threadIdx.x; p < pairs; p += blockDim.x) atomicAdd(&count[chosen[p]], 1);
+    for (int p = threadIdx.x; p < pairs; p += blockDim.x) {
+        const int e = chosen[p];
+        if (e < experts) atomicAdd(&count[e], 1);
+    }
     __syncthreads();
     if (threadIdx.x == 0) {
         int rows = 0, tl = 0;
@@ -233,6 +259,10 @@ moe_sort_kernel(const int32_t* __restrict__ chosen, int pairs, int experts, int 
     __syncthreads();
     for (int p = threadIdx.x; p < pairs; p += blockDim.x) {
         const int e = chosen[p];
+        if (e >= experts) {
+            place_of_pair[p] = -1;
+            continue;
+        }
         const int at = first[e] + atomicAdd(&count[e], 1);
         pair_token[at] = p / top;
         place_of_pair[p] = at;
@@ -433,27 +463,63 @@ moe_expert_mfma_kernel(const bf16_t* __restrict__ x, const int32_t* __restrict__
         }
 }
 
-// out[t][c] = sum_j weight[t][j] y[place[t top + j]][c] (weight null: every weight one) + sum of the slabs of shared[t][c]
+// A logit that weighs the shared expert's result, by its sigmoid: float32 at column `column` of rows of `stride` (slabs added in
+// order); z null: none, the result as it is.
+struct SharedGate {
+    const float* z;
+    int parts;
+    size_t part_stride;
+    int stride, column;
+};
+
+__device__ __forceinline__ float shared_weight(const SharedGate& g, int t) {
+    if (g.z == nullptr) return 1.0f;
+    const float* at = g.z + (size_t)t * g.stride + g.column;
+    float v = at[0];
+    for (int q = 1; q < g.parts; ++q) v += at[q * g.part_stride];
+    return 1.0f / (1.0f + expf(-v));
+}
+
+// out[t][c] = sum_j weight[t][j] y[place[t top + j]][c] (weight null: every weight one; place below 0: x[t][c] in the place of
+// y's row) + the shared gate's weight times the sum of the slabs of shared[t][c]
+template <typename TX>
 __global__ void moe_combine_kernel(const float* __restrict__ y, const int32_t* __restrict__ place, const float* __restrict__ weight,
-                                   const float* __restrict__ shared, int shared_parts, size_t shared_stride,
-                                   float* __restrict__ out, int tokens, int width, int top) {
+                                   const float* __restrict__ shared, int shared_parts, size_t shared_stride, const TX* __restrict__ x,
+                                   SharedGate gate, float* __restrict__ out, int tokens, int width, int top) {
     const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
     if (i >= (size_t)tokens * width) return;
     const int t = (int)(i / width), c = (int)(i - (size_t)t * width);
     float acc = 0.0f;
-    for (int j = 0; j < top; ++j)
-        acc = fmaf(weight != nullptr ? weight[(size_t)t * top + j] : 1.0f, y[(size_t)place[(size_t)t * top + j] * width + c], acc);
-    for (int p = 0; p < shared_parts; ++p) acc += shared[p * shared_stride + i];
+    for (int j = 0; j < top; ++j) {
+        const int at = place[(size_t)t * top + j];
+        const float v = at >= 0 ? y[(size_t)at * width + c] : (x != nullptr ? load_f(x, i) : 0.0f);
+        acc = fmaf(weight != nullptr ? weight[(size_t)t * top + j] : 1.0f, v, acc);
+    }
+    if (shared_parts > 0) {
+        float a = 0.0f;
+        for (int p = 0; p < shared_parts; ++p) a += shared[p * shared_stride + i];
+        acc = fmaf(shared_weight(gate, t), a, acc);
+    }
     out[i] = acc;
 }
 
+__device__ __forceinline__ float4 row4(const float* x, size_t i4) { return ((const float4*)x)[i4]; }
+__device__ __forceinline__ float4 row4(const bf16_t* x, size_t i4) {
+    const uint2 r = ((const uint2*)x)[i4];
+    return make_float4(__uint_as_float(r.x << 16), __uint_as_float(r.x & 0xffff0000u), __uint_as_float(r.y << 16), __uint_as_float(r.y & 0xffff0000u));
+}
+
 // The same four columns a thread, for widths that are a multiple of 4: blockIdx.x a token, its rows of y asked for eight at a time.
+template <typename TX>
 __global__ void __launch_bounds__(256)
 moe_combine4_kernel(const float* __restrict__ y, const int32_t* __restrict__ place, const float* __restrict__ weight,
-                    const float* __restrict__ shared, int shared_parts, size_t shared_stride, float* __restrict__ out, int width, int top) {
+                    const float* __restrict__ shared, int shared_parts, size_t shared_stride, const TX* __restrict__ x, SharedGate gate,
+                    float* __restrict__ out, int width, int top) {
     const int t = blockIdx.x, c4 = blockIdx.y * 256 + threadIdx.x, w4 = width / 4;
     if (c4 >= w4) return;
+    const size_t at = (size_t)t * w4 + c4;
     float4 acc = make_float4(0.0f, 0.0f, 0.0f, 0.0f);
+    const float4 own = x != nullptr ? row4(x, at) : acc;
     for (int j0 = 0; j0 < top; j0 += 8) {
         float4 v[8];
         float by[8];
@@ -461,8 +527,9 @@ moe_combine4_kernel(const float* __restrict__ y, const int32_t* __restrict__ pla
         for (int j = 0; j < 8; ++j)
             if (j0 + j < top) {
                 const size_t pair = (size_t)t * top + j0 + j;
+                const int from = place[pair];
                 by[j] = weight != nullptr ? weight[pair] : 1.0f;
-                v[j] = ((const float4*)y)[(size_t)place[pair] * w4 + c4];
+                v[j] = from >= 0 ? ((const float4*)y)[(size_t)from * w4 + c4] : own;
             }
 #pragma unroll
         for (int j = 0; j < 8; ++j)
@@ -473,10 +540,17 @@ moe_combine4_kernel(const float* __restrict__ y, const int32_t* __restrict__ pla
                 acc.w = fmaf(by[j], v[j].w, acc.w);
             }
     }
-    const size_t at = (size_t)t * w4 + c4;
-    for (int p = 0; p < shared_parts; ++p) {
-        const float4 s = ((const float4*)(shared + p * shared_stride))[at];
-        acc.x += s.x; acc.y += s.y; acc.z += s.z; acc.w += s.w;
+    if (shared_parts > 0) {
+        float4 a = make_float4(0.0f, 0.0f, 0.0f, 0.0f);
+        for (int p = 0; p < shared_parts; ++p) {
+            const float4 s = ((const float4*)(shared + p * shared_stride))[at];
+            a.x += s.x; a.y += s.y; a.z += s.z; a.w += s.w;
+        }
+        const float by = shared_weight(gate, t);
+        acc.x = fmaf(by, a.x, acc.x);
+        acc.y = fmaf(by, a.y, acc.y);
+        acc.z = fmaf(by, a.z, acc.z);
+        acc.w = fmaf(by, a.w, acc.w);
     }
     ((float4*)out)[at] = acc;
 }
@@ -496,22 +570,25 @@ extern "C" int kipp_moe_route(const float* z, int parts, int stride, int32_t* ch
     return KIPP_LAUNCH_CHECK();
 }
 
-// The same with sigmoid scores, a correction of the choice (or none) and groups of which `group_keep` of `group_count` stay.
+// The same with sigmoid scores (`softmax` 0) or a softmax, a correction of the choice (or none) and groups of which `group_keep` of
+// `group_count` stay, by the sum of their two largest choice scores (`by_largest` 0) or their largest.  `experts` counts the
+// router's outputs, the last `identity` of which are identity experts.
 extern "C" int kipp_moe_route_grouped(const float* z, int parts, int stride, const float* correction, int32_t* chosen, float* weight,
                                       int tokens, int experts, int top, float eps, int group_count, int group_keep, float scale,
-                                      int renormalize, int32_t* pair_token, int32_t* place_of_pair, int32_t* tiles, int max_tiles, int tile_rows,
-                                      float* row_weight, hipStream_t stream) {
+                                      int renormalize, int softmax, int by_largest, int identity, int32_t* pair_token, int32_t* place_of_pair,
+                                      int32_t* tiles, int max_tiles, int tile_rows, float* row_weight, hipStream_t stream) {
     if (tokens <= 0) return 0;
+    if (identity < 0 || identity >= experts || (identity > 0 && row_weight != nullptr)) return -1;
     if (experts <= 0 || experts > MAX_EXPERTS || top <= 0 || top > MAX_TOP || top > experts || stride < experts || parts <= 0) return -1;
     if (group_count <= 0 || experts % group_count || group_keep <= 0 || group_keep > group_count ||
         top > group_keep * (experts / group_count)) return -1;
-    const int pairs = tokens * top;
+    const int pairs = tokens * top, real = experts - identity;
     if (tile_rows != TILE_ROWS && tile_rows != MFMA_ROWS) return -1;
-    if (max_tiles < (pairs + tile_rows - 1) / tile_rows + (experts < pairs ? experts : pairs)) return -1;
+    if (max_tiles < (pairs + tile_rows - 1) / tile_rows + (real < pairs ? real : pairs)) return -1;
     hipLaunchKernelGGL(moe_route_grouped_kernel, dim3((tokens + ROUTE_WAVES - 1) / ROUTE_WAVES), dim3(ROUTE_WAVES * KIPP_WAVE), 0, stream, z,
                        parts, (size_t)tokens * stride, stride, correction, chosen, weight, tokens, experts, top, eps, group_count, group_keep,
-                       scale, renormalize);
-    hipLaunchKernelGGL(moe_sort_kernel, dim3(1), dim3(1024), 0, stream, (const int32_t*)chosen, pairs, experts, top, pair_token,
+                       scale, renormalize, softmax, by_largest);
+    hipLaunchKernelGGL(moe_sort_kernel, dim3(1), dim3(1024), 0, stream, (const int32_t*)chosen, pairs, real, top, pair_token,
                        place_of_pair, tiles, max_tiles, tile_rows, (const float*)weight, row_weight);
     return KIPP_LAUNCH_CHECK();
 }
@@ -564,17 +641,30 @@ extern "C" int kipp_moe_expert_gated(const void* x, int x_dtype, const int32_t* 
     return launch_expert<true>(x, x_dtype, gather, row_weight, w, w_dtype, tiles, max_tiles, out, out_dtype, n_out, k, act, tile_rows, stream);
 }
 
+// `x` (or null): the rows that identity experts hand on.  `gate_z` (or null): rows whose column `gate_column` holds the logit that
+// weighs `shared` (float32, or slabs of it).
 extern "C" int kipp_moe_combine(const float* y, const int32_t* place, const float* weight, const float* shared, int shared_parts,
+                                const void* x, int x_dtype, const float* gate_z, int gate_parts, int gate_stride, int gate_column,
                                 float* out, int tokens, int width, int top, hipStream_t stream) {
     if (tokens <= 0) return 0;
+    if (width <= 0 || top <= 0 || (x_dtype != KIPP_F32 && x_dtype != KIPP_BF16)) return -1;
+    if (gate_z != nullptr && (gate_parts <= 0 || gate_column < 0 || gate_column >= gate_stride || shared == nullptr)) return -1;
     const size_t total = (size_t)tokens * width;
-    if (width % 4 == 0 && (((uintptr_t)y | (uintptr_t)out | (uintptr_t)shared) & 15) == 0) {
-        hipLaunchKernelGGL(moe_combine4_kernel, dim3(tokens, (width / 4 + 255) / 256), dim3(256), 0, stream, y, place, weight, shared,
-                           shared != nullptr ? shared_parts : 0, total, out, width, top);
+    const SharedGate gate = {gate_z, gate_parts, (size_t)tokens * gate_stride, gate_stride, gate_column};
+    const int parts = shared != nullptr ? shared_parts : 0;
+    if (width % 4 == 0 && (((uintptr_t)y | (uintptr_t)out | (uintptr_t)shared | (uintptr_t)x) & 15) == 0) {
+        dim3 grid(tokens, (width / 4 + 255) / 256), block(256);
+        if (x_dtype == KIPP_BF16)
+            hipLaunchKernelGGL(moe_combine4_kernel<bf16_t>, grid, block, 0, stream, y, place, weight, shared, parts, total, (const bf16_t*)x, gate, out, width, top);
+        else
+            hipLaunchKernelGGL(moe_combine4_kernel<float>, grid, block, 0, stream, y, place, weight, shared, parts, total, (const float*)x, gate, out, width, top);
         return KIPP_LAUNCH_CHECK();
     }
-    hipLaunchKernelGGL(moe_combine_kernel, dim3((unsigned)((total + 255) / 256)), dim3(256), 0, stream, y, place, weight, shared,
-                       shared != nullptr ? shared_parts : 0, total, out, tokens, width, top);
+    dim3 grid((unsigned)((total + 255) / 256)), block(256);
+    if (x_dtype == KIPP_BF16)
+        hipLaunchKernelGGL(moe_combine_kernel<bf16_t>, grid, block, 0, stream, y, place, weight, shared, parts, total, (const bf16_t*)x, gate, out, tokens, width, top);
+    else
+        hipLaunchKernelGGL(moe_combine_kernel<float>, grid, block, 0, stream, y, place, weight, shared, parts, total, (const float*)x, gate, out, tokens, width, top);
     return KIPP_LAUNCH_CHECK();
 }
 

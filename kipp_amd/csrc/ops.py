@@ -159,6 +159,30 @@ def rmsnorm_scaled_delta(x: torch.Tensor, delta: torch.Tensor, dscale: torch.Ten
     return out
 
 
+def normed_sum_step(x: torch.Tensor, terms, next_w: Optional[torch.Tensor] = None, next_eps: float = 0.0,
+                    out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """x += sum over `terms` of scale * rmsnorm(delta) * weight in place (float32 [rows, width]); with `out`, out =
+    rmsnorm(x) * next_w in out's type, in the same kernel.  `terms`: one or two of (delta, weight, eps, scale), delta float32
+    [rows, width] or slabs of it."""
+    rows, width = x.shape
+    _need(x.dtype == torch.float32 and len(terms) in (1, 2), "normed_sum_step: float32 x, one or two terms")
+    args = []
+    for delta, weight, eps, scale in terms:
+        _dev(x, delta, weight)
+        parts, r, w = _slabs(delta, "normed_sum_step")
+        _need((r, w) == (rows, width) and weight.dtype == torch.float32 and weight.numel() == width, "normed_sum_step: deltas of x's shape, float32 weights [width]")
+        args += [_ptr(delta), parts, _ptr(weight), float(eps), float(scale)]
+    if len(terms) == 1:
+        args += [None, 0, None, 0.0, 0.0]
+    _dev(x, next_w, out)
+    _need(out is None or (out.shape == x.shape and next_w is not None and next_w.dtype == torch.float32 and next_w.numel() == width),
+          "normed_sum_step: out has x's shape and needs the next norm's float32 weight")
+    fn = _fn("elementwise", "kipp_normed_sum_step", [_c_ptr] + [_c_ptr, _c_int, _c_ptr, _c_float, _c_float] * 2
+             + [_c_ptr, _c_float, _c_ptr, _c_int, _c_int, _c_int, _c_ptr])
+    _check(fn(_ptr(x), *args, _ptr(next_w), float(next_eps), _ptr(out), _code(out) if out is not None else F32, rows, width, _stream()), "normed_sum_step")
+    return x
+
+
 def scale_columns(delta: torch.Tensor, scale: torch.Tensor, x: torch.Tensor, add: bool = False) -> torch.Tensor:
     """x[r, c] = scale[c] * delta[r, c] (float32; `delta` may come in slabs), or with `add` x[r, c] += that."""
     _dev(x, delta, scale)
@@ -436,14 +460,17 @@ def head_prepare(proj: torch.Tensor, q_out: torch.Tensor, k_cache: torch.Tensor,
                  temp_coef: float = 0.0, temp_every: int = 0, write_kv: bool = True,
                  q_head_scale: Optional[torch.Tensor] = None, v_norm_eps: Optional[float] = None,
                  angles: Optional[torch.Tensor] = None, rotary_dim: int = 0, v_first_in: Optional[torch.Tensor] = None,
-                 v_first_out: Optional[torch.Tensor] = None, v_lambda: Optional[torch.Tensor] = None) -> torch.Tensor:
+                 v_first_out: Optional[torch.Tensor] = None, v_lambda: Optional[torch.Tensor] = None, interleaved: bool = False,
+                 keys_as_values: bool = False) -> torch.Tensor:
     """From a step's input product `proj` (float32 [tokens, >= n_q d + n_kv d + n_kv dv], columns q | k | v | ..., or slabs
     of it): `bias` added (float32 over the q | k | v columns), every head of q and k RMS-normed (`norm`: "none", "plain"
     or "weighted" with `q_norm_w` / `k_norm_w` [d]), queries at position p times 1 + temp_coef ln(floor((p + 1) /
     temp_every) + 1) (temp_every 0: none), queries of head h times `q_head_scale[h]` (float32 [n_q]), every value head over
     its root mean square with `v_norm_eps` inside the root (None: values as they are), q kept in `q_out`, k and v written
     into the pages of their positions.  `angles` (`rotary_angles`, float32 [tokens, rotary_dim]): after the norm the first
-    `rotary_dim` numbers of every q and k head are turned, number i with number i + rotary_dim / 2.  `v_first_out` (float32
+    `rotary_dim` numbers of every q and k head are turned, number i with number i + rotary_dim / 2 (`interleaved`: number 2i with
+    number 2i + 1).  `keys_as_values`: there are no value columns; a value is its key as projected (with its bias, before norm and
+    rotation; dv = d).  `v_first_out` (float32
     [tokens, n_kv dv]) receives the values as they are; with `v_first_in` (another layer's, of the same tokens) and `v_lambda`
     (float32, one number on the device) the value that is cached is (1 - lambda) v + lambda v_first."""
     _dev(proj, q_out, k_cache, v_cache, positions, seq_of_token, block_table, bias, q_norm_w, k_norm_w, q_head_scale, angles,
@@ -463,12 +490,15 @@ def head_prepare(proj: torch.Tensor, q_out: torch.Tensor, k_cache: torch.Tensor,
     for t, name in ((positions, "positions"), (seq_of_token, "seq_of_token"), (block_table, "block_table")):
         _i32(t, name)
     parts, n, stride = _slabs(proj, "head_prepare")
+    _need(not keys_as_values or (d == dv and v_first_in is None and v_first_out is None and v_norm_eps is None),
+          "head_prepare: keys that are the values are as wide as them, without value norm or mixing")
+    kv_columns = n_kv * d + (0 if keys_as_values else n_kv * dv)
     _need(norm in ("none", "plain", "weighted"), "head_prepare: norm is one of none, plain, weighted")
-    _need(stride >= n_q * d + (n_kv * d + n_kv * dv if write_kv else 0), "head_prepare: the projections are narrower than q, k and v")
+    _need(stride >= n_q * d + (kv_columns if write_kv else 0), "head_prepare: the projections are narrower than q, k and v")
     _need(0 < d <= 256 and 0 < dv <= 256, "head_prepare: head sizes from 1 to 256")
     _need(q_out.shape == (n, n_q * d) and positions.numel() == n and seq_of_token.numel() == n, "head_prepare: one row a token")
     if bias is not None:
-        _need(bias.dtype == torch.float32 and bias.numel() == n_q * d + n_kv * d + n_kv * dv, "head_prepare: float32 bias over q | k | v")
+        _need(bias.dtype == torch.float32 and bias.numel() == n_q * d + kv_columns, "head_prepare: float32 bias over q | k | v")
     if norm == "weighted":
         _need(q_norm_w is not None and k_norm_w is not None and q_norm_w.dtype == k_norm_w.dtype == torch.float32
               and q_norm_w.numel() == d and k_norm_w.numel() == d, "head_prepare: float32 norm weights [d]")
@@ -478,13 +508,15 @@ def head_prepare(proj: torch.Tensor, q_out: torch.Tensor, k_cache: torch.Tensor,
     _need(block_table.dim() == 2 and int(temp_every) >= 0, "head_prepare: block_table is [sequences, blocks]")
     fn = _fn("head_prepare", "kipp_head_prepare_rotated",
              [_c_ptr, _c_int, _c_int, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int,
-              _c_int, _c_ptr, _c_ptr, _c_float, _c_float, _c_int] + [_c_int] * 7 + [_c_ptr, _c_float, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr])
+              _c_int, _c_ptr, _c_ptr, _c_float, _c_float, _c_int] + [_c_int] * 7
+             + [_c_ptr, _c_float, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_ptr])
     _check(fn(_ptr(proj), parts, stride, _ptr(bias), _ptr(q_out), _code(q_out), _ptr(k_cache), _ptr(v_cache), _code(k_cache),
               _ptr(positions), _ptr(seq_of_token), _ptr(block_table), block_table.shape[1],
               {"none": 0, "plain": 1, "weighted": 2}[norm], _ptr(q_norm_w), _ptr(k_norm_w), float(eps), float(temp_coef),
               int(temp_every), n, n_q, n_kv, d, dv, k_cache.shape[2], int(write_kv), _ptr(q_head_scale),
               -1.0 if v_norm_eps is None else float(v_norm_eps), _ptr(angles), int(rotary_dim) if angles is not None else 0,
-              _ptr(v_first_in), _ptr(v_first_out), _ptr(v_lambda), v_cache.shape[3], _stream()), "head_prepare")
+              _ptr(v_first_in), _ptr(v_first_out), _ptr(v_lambda), v_cache.shape[3], int(bool(interleaved)), int(bool(keys_as_values)), _stream()),
+           "head_prepare")
     return q_out
 
 
@@ -970,35 +1002,41 @@ def moe_max_tiles(tokens: int, experts: int, top: int, tile_rows: int = 16) -> i
 def moe_route(z: torch.Tensor, experts: int, top: int, eps: float, chosen: torch.Tensor, weight: torch.Tensor,
               pair_token: torch.Tensor, place_of_pair: torch.Tensor, tiles: torch.Tensor, tile_rows: int = 16,
               router: str = "softmax", correction: Optional[torch.Tensor] = None, groups: Optional[tuple] = None, scale: float = 1.0,
-              renormalize: bool = True, row_weight: Optional[torch.Tensor] = None):
+              renormalize: bool = True, row_weight: Optional[torch.Tensor] = None, identity: int = 0, group_score: str = "top2"):
     """From router logits `z` (float32 [tokens, >= experts] or slabs): softmax over the experts, the `top` largest a token
     (`chosen`, int32 [tokens, top]) with weights p / (sum of the chosen p + eps) (`weight`, float32 [tokens, top]); then the
     pairs sorted by expert: `pair_token` [pairs] the token of every sorted row, `place_of_pair` [pairs] the row of pair
     (token, choice), `tiles` int32 [max_tiles, 3] = (expert, first row, rows) of up to `tile_rows` rows, unused tiles with 0 rows.
+    `router` "sigmoid": sigmoid scores in the softmax's place.  `correction` (float32 [experts + identity]) is added to the scores
+    for the choice alone; `groups` (count, keep): only experts of the `keep` best of `count` equal groups of neighbours can be chosen,
+    a group's score the sum of its two largest choice scores (`group_score` "top2") or its largest ("top1"); weights times `scale`.
     `renormalize` False (sigmoid router): weights are the scores themselves times `scale`.  `row_weight` (float32 [pairs]) receives
-    every sorted row's weight."""
+    every sorted row's weight.  `identity` I: the router has I outputs behind the experts' that are identity experts; a pair that
+    chose one has no sorted row and place -1."""
     _dev(z, chosen, weight, pair_token, place_of_pair, tiles, row_weight)
     parts, n, stride = _slabs(z, "moe_route")
+    real, experts = experts, experts + int(identity)
     for t, name in ((chosen, "chosen"), (pair_token, "pair_token"), (place_of_pair, "place_of_pair"), (tiles, "tiles")):
         _i32(t, name)
-    _need(0 < top <= experts <= 1024 and top <= 32 and stride >= experts, "moe_route: up to 1,024 experts, up to 32 a token")
+    _need(0 < top <= experts <= 1024 and top <= 32 and stride >= experts and real > 0 and identity >= 0, "moe_route: up to 1,024 experts, up to 32 a token")
+    _need(group_score in ("top1", "top2") and not (identity and row_weight is not None), "moe_route: group_score is top1 or top2; no row weights with identity experts")
     _need(chosen.shape == (n, top) and weight.shape == (n, top) and weight.dtype == torch.float32 and pair_token.numel() == n * top
-          and place_of_pair.numel() == n * top and tiles.dim() == 2 and tiles.shape[1] == 3 and tiles.shape[0] >= moe_max_tiles(n, experts, top, tile_rows),
+          and place_of_pair.numel() == n * top and tiles.dim() == 2 and tiles.shape[1] == 3 and tiles.shape[0] >= moe_max_tiles(n, real, top, tile_rows),
           "moe_route: output shapes")
     _need(router in ("softmax", "sigmoid"), "moe_route: router is softmax or sigmoid")
     _need(row_weight is None or (row_weight.dtype == torch.float32 and row_weight.numel() == n * top), "moe_route: row_weight is float32 [pairs]")
-    if router == "sigmoid":
+    _need(renormalize or router == "sigmoid", "moe_route: weights as they are belong to the sigmoid router")
+    if router == "sigmoid" or correction is not None or groups is not None or scale != 1.0 or identity:
         _dev(correction)
         count, keep = groups if groups is not None else (1, 1)
         _need(correction is None or (correction.dtype == torch.float32 and correction.numel() == experts), "moe_route: float32 correction [experts]")
         _need(count > 0 and experts % count == 0 and 0 < keep <= count and top <= keep * (experts // count),
               "moe_route: equal groups, of which at least one stays, with experts enough for a token's choice")
         fn = _fn("moe", "kipp_moe_route_grouped", [_c_ptr, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_float, _c_int, _c_int, _c_float,
-                                                   _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr, _c_ptr])
+                                                   _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr, _c_ptr])
         _check(fn(_ptr(z), parts, stride, _ptr(correction), _ptr(chosen), _ptr(weight), n, experts, top, float(eps), int(count), int(keep), float(scale),
-                  int(bool(renormalize)), _ptr(pair_token), _ptr(place_of_pair), _ptr(tiles), tiles.shape[0], int(tile_rows), _ptr(row_weight), _stream()), "moe_route")
+                  int(bool(renormalize)), int(router == "softmax"), int(group_score == "top1"), int(identity), _ptr(pair_token), _ptr(place_of_pair), _ptr(tiles), tiles.shape[0], int(tile_rows), _ptr(row_weight), _stream()), "moe_route")
         return chosen, weight
-    _need(correction is None and groups is None and scale == 1.0 and renormalize, "moe_route: correction, groups, scale and weights as they are belong to the sigmoid router")
     fn = _fn("moe", "kipp_moe_route", [_c_ptr, _c_int, _c_int, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_float, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr, _c_ptr])
     _check(fn(_ptr(z), parts, stride, _ptr(chosen), _ptr(weight), n, experts, top, float(eps), _ptr(pair_token), _ptr(place_of_pair), _ptr(tiles),
               tiles.shape[0], int(tile_rows), _ptr(row_weight), _stream()), "moe_route")
@@ -1048,10 +1086,12 @@ def moe_expert_gated(x: torch.Tensor, gather: Optional[torch.Tensor], row_weight
     return out
 
 
-def moe_combine(y: torch.Tensor, place_of_pair: torch.Tensor, weight: Optional[torch.Tensor], shared: Optional[torch.Tensor], out: torch.Tensor) -> torch.Tensor:
+def moe_combine(y: torch.Tensor, place_of_pair: torch.Tensor, weight: Optional[torch.Tensor], shared: Optional[torch.Tensor], out: torch.Tensor,
+                identity_rows: Optional[torch.Tensor] = None, shared_gate: Optional[tuple] = None) -> torch.Tensor:
     """out[t] = sum_j weight[t, j] y[place_of_pair[t top + j]] + shared[t] (float32; `weight` None: every weight is one; `shared`
-    may come in slabs or be None)."""
-    _dev(y, place_of_pair, weight, shared, out)
+    may come in slabs or be None).  `identity_rows` [tokens, width]: what stands in for y's row where a place is -1 (None: nothing
+    is added there).  `shared_gate` (z, column): shared[t] is multiplied by sigmoid(z[t, column]), z float32 rows or slabs of them."""
+    _dev(y, place_of_pair, weight, shared, out, identity_rows)
     _i32(place_of_pair, "place_of_pair")
     n, width = out.shape
     top = place_of_pair.numel() // max(n, 1)
@@ -1062,8 +1102,17 @@ def moe_combine(y: torch.Tensor, place_of_pair: torch.Tensor, weight: Optional[t
     if shared is not None:
         parts, rows, w2 = _slabs(shared, "moe_combine")
         _need((rows, w2) == (n, width), "moe_combine: shared is [tokens, width] or slabs of it")
-    fn = _fn("moe", "kipp_moe_combine", [_c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_int, _c_int, _c_int, _c_ptr])
-    _check(fn(_ptr(y), _ptr(place_of_pair), _ptr(weight), _ptr(shared), parts, _ptr(out), n, width, top, _stream()), "moe_combine")
+    _need(identity_rows is None or tuple(identity_rows.shape) == (n, width), "moe_combine: identity rows are [tokens, width]")
+    gate_z, gate_parts, gate_stride, gate_column = None, 0, 0, 0
+    if shared_gate is not None:
+        gate_z, gate_column = shared_gate
+        _dev(gate_z)
+        gate_parts, rows, gate_stride = _slabs(gate_z, "moe_combine")
+        _need(rows == n and 0 <= gate_column < gate_stride and shared is not None, "moe_combine: the gate is a column of logits, one row a token")
+    fn = _fn("moe", "kipp_moe_combine", [_c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_int, _c_ptr, _c_int, _c_int, _c_int, _c_ptr, _c_int, _c_int,
+                                         _c_int, _c_ptr])
+    _check(fn(_ptr(y), _ptr(place_of_pair), _ptr(weight), _ptr(shared), parts, _ptr(identity_rows), _code(identity_rows) if identity_rows is not None else F32,
+              _ptr(gate_z), gate_parts, gate_stride, int(gate_column), _ptr(out), n, width, top, _stream()), "moe_combine")
     return out
 
 
@@ -1727,7 +1776,47 @@ def gemm_skinny_swiglu(x: torch.Tensor, w_gate_up: torch.Tensor, out: torch.Tens
     return out
 
 
-TILES_END = {"slabs": 0, "swiglu": 1, "bf16": 2}
+def gemm_skinny_relu2(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, tiles: torch.Tensor = None, row_scale=None,
+                      x_steps_major: bool = False, out_steps_major: bool = False) -> torch.Tensor:
+    """out[M, N] (bfloat16) = relu(x . w^T)^2 for M <= 64 rows; `tiles` = tile_weight(w).  `row_scale`, `x_steps_major`: as in
+    `gemm_skinny` (the product is scaled before the activation); `out_steps_major`: `out` is written in the order of
+    `steps_major` (N a multiple of 32)."""
+    _dev(x, w, out)
+    m, k = x.shape
+    n = w.shape[0]
+    _need(x.dtype == torch.bfloat16 and w.dtype == torch.bfloat16 and out.dtype == torch.bfloat16, "gemm_skinny_relu2: bfloat16 operands and output")
+    _need(w.shape == (n, k) and out.shape == (m, n), "gemm_skinny_relu2: shapes do not match")
+    _need(gemm_skinny_ok(m, k), "gemm_skinny_relu2: at most 64 rows, K a multiple of 8 and at least 32")
+    _need((not x_steps_major or k % 32 == 0) and (not out_steps_major or n % 32 == 0),
+          "gemm_skinny_relu2: rows in steps-major order need their width to be a multiple of 32")
+    tiled = _tiles_ok(tiles, n, k, "gemm_skinny_relu2")
+    sumsq, sumsq_parts, eps = _row_scale_args(row_scale, m, "gemm_skinny_relu2")
+    fn = _fn("gemm_skinny", "kipp_gemm_skinny_relu2",
+             [_c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_int, _c_float, _c_int, _c_int, _c_ptr])
+    _check(fn(_ptr(x), _ptr(tiles if tiled else w), _ptr(out), m, n, k, tiled, sumsq, sumsq_parts, eps,
+              int(bool(x_steps_major)), int(bool(out_steps_major)), _stream()), "gemm_skinny_relu2")
+    return out
+
+
+def gemm_rows_relu2_pays(m: int, n: int, k: int) -> bool:
+    """Whether, for this shape, the product that ends in the square of relu is taken over a split product and an activation kernel."""
+    return bool(build.library("gemm_rows").kipp_gemm_rows_relu2_pays(int(m), int(n), int(k)))
+
+
+def gemm_rows_relu2(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, tiles: torch.Tensor = None, cut: int = 0) -> torch.Tensor:
+    """out[M, N] (bfloat16) = relu(x . w^T)^2 for a few dozen rows (up to 256); `tiles` = tile_weight(w); `cut` as in `gemm_rows`."""
+    _dev(x, w, out)
+    m, k = x.shape
+    n = w.shape[0]
+    _need(x.dtype == w.dtype == out.dtype == torch.bfloat16 and w.shape == (n, k) and out.shape == (m, n) and gemm_rows_ok(m, k),
+          "gemm_rows_relu2: bfloat16 x [M, K], w [N, K], out [M, N], up to 256 rows, K a multiple of 8 and at least 32")
+    tiled = _tiles_ok(tiles, n, k, "gemm_rows_relu2")
+    fn = _fn("gemm_rows", "kipp_gemm_rows_relu2", [_c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr])
+    _check(fn(_ptr(x), _ptr(tiles if tiled else w), _ptr(out), m, n, k, tiled, int(cut), _stream()), "gemm_rows_relu2")
+    return out
+
+
+TILES_END = {"slabs": 0, "swiglu": 1, "bf16": 2, "relu2": 3}
 
 
 def gemm_tiles_ok(m: int, k: int, n: int = 1) -> bool:
@@ -1745,7 +1834,7 @@ def gemm_tiles(x: torch.Tensor, w: torch.Tensor, end: str = "slabs", max_parts: 
     """x [M, K] . w [N, K]^T on the matrix cores for many rows, bfloat16 operands, float32 accumulation.
     end "slabs": float32 [parts, M, N] whose sum over parts is the product (parts <= max_parts, chosen from the shape);
     "swiglu": w = [gate; up] of [2 I, K], the result is bfloat16 [M, I] = silu(x . gate^T) * (x . up^T);
-    "bf16": bfloat16 [M, N].  `force` = 100 wm + 10 wn + parts (+ 1000: workgroups of 8 waves, four across, wave tiles
+    "bf16": bfloat16 [M, N]; "relu2": bfloat16 [M, N] = relu(x . w^T)^2.  `force` = 100 wm + 10 wn + parts (+ 1000: workgroups of 8 waves, four across, wave tiles
     4 x 2 or 2 x 2; + 2000, bfloat16 ends: those for the whole rounds of 256 tiles and smaller tiles for the columns
     that are left, 8 waves on half the rows or, + 10000 r, 4 waves on 256 x 64, 128 x 128 or 128 x 64 outputs) takes
     that cut instead of the planned one (the runtime's timed choice, tests)."""

@@ -57,6 +57,13 @@ class PreNormBlock:
         return self.parts[role].apply(delta) if role in self.parts else delta
 
 
+@register("block", "pre_norm_mixer")
+class PreNormMixerBlock(PreNormBlock):
+    """The first half of the pre-norm arrangement alone: a layer without a feed-forward."""
+
+    roles = (("mixer_norm", "norm"), ("mixer", "mixer"))
+
+
 @register("block", "scaled_pre_norm")
 class ScaledPreNormBlock(PreNormBlock):
     """The pre-norm arrangement with a scale on every sublayer's result: x += mixer_scale(mixer(mixer_norm(x)));

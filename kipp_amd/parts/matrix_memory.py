@@ -89,6 +89,7 @@ class DecayAttention:
 @register("mixer", "gated_delta")
 class GatedDelta:
     graph_safe = True   # forward launches kernels only: no host reads, no data-dependent launches
+    takes_scaled_rows = True
 
     def __init__(self, spec, runtime):
         self.spec = spec

@@ -22,7 +22,7 @@ import math
 import torch
 
 from ..cache.needs import KVNeed
-from .base import ParamSpec, build_part, register
+from .base import ParamSpec, build_part, part_class, part_params, register
 
 
 
@@ -55,9 +55,10 @@ class Attention:
         p = {q: ParamSpec((spec.q_dim, spec.hidden_size)), o: ParamSpec((spec.hidden_size, spec.out_dim))}
         if spec.own_kv:
             p[k] = ParamSpec((spec.kv_dim, spec.hidden_size))
-            p[v] = ParamSpec((spec.v_dim, spec.hidden_size))
+            if not spec.keys_as_values:
+                p[v] = ParamSpec((spec.v_dim, spec.hidden_size))
         if spec.bias:
-            for name, width in zip(spec.bias_names, (spec.q_dim, spec.kv_dim, spec.v_dim)):
+            for name, width in list(zip(spec.bias_names, (spec.q_dim, spec.kv_dim, spec.v_dim)))[:2 if spec.keys_as_values else 3]:
                 if spec.own_kv or name == spec.bias_names[0]:
                     p[name] = ParamSpec((width,), "float", ("normal", 0.1))
         if spec.qk_norm_eps is not None and spec.qk_norm_weight:
@@ -100,7 +101,7 @@ class Attention:
         import torch
         s = self.spec
         names = s.names
-        rows = [tensors[names[0]]] + ([tensors[names[1]], tensors[names[2]]] if s.own_kv else [])
+        rows = [tensors[name] for name in names[:1 if not s.own_kv else (2 if s.keys_as_values else 3)]]
         if len({t.dtype for t in rows}) > 1:
             rows = [t.float() for t in rows]
         # rows concatenated: one product serves q, k and v; no output element changes
@@ -122,7 +123,7 @@ class Attention:
             self.head_temp_capped = ((self.head_temp.float() if self.head_temp is not None else ones) * (self.scale / s.softcap)).contiguous()
         self.bias = None
         if s.bias:
-            held = [tensors[name] for name in (s.bias_names if s.own_kv else s.bias_names[:1])]
+            held = [tensors[name] for name in s.bias_names[:1 if not s.own_kv else (2 if s.keys_as_values else 3)]]
             if not s.own_kv:        # the kernel's bias runs over q | k | v: nothing is added where nothing is written
                 held.append(torch.zeros(s.kv_dim + s.v_dim, dtype=torch.float32, device=held[0].device))
             self.bias = torch.cat([t.float() for t in held]).contiguous()
@@ -200,22 +201,20 @@ class Attention:
     def _forward_prepared(self, x, batch, cache):
         """The mixer with any of: biases, a norm without weights, a factor on the queries that grows with the position,
         values of their own width, keys and values of another run, chunks, the added one in the softmax's denominator,
-        values mixed with an earlier run's, a bias on the output.  One kernel makes the heads ready from the input product
+        values mixed with an earlier run's, keys that are the values, a bias on the output.  One kernel makes the heads ready from the input product
         (and turns them, where the mixer rotates); the attention kernels are the same."""
         s, rt = self.spec, self.rt
         from ..runtime import WeightedDelta
         inv_freq, rotary_dim = self.position.rotary_table()
         angles = None
         if inv_freq is not None:
-            if getattr(self.position, "pairing", "half") != "half":
-                raise NotImplementedError("the kernel that makes these heads ready turns halves of a head, not neighbours")
             angles = self.position.angles(batch)
         n = x.shape[0]
         table = batch.block_tables[cache.group]
         d, dv = s.head_dim, s.value_dim
         if not s.own_kv and cache.writable:
             raise ValueError("an attention mixer without key and value projections needs the cache of another run")
-        proj = rt.linear(rt.rows_of(x), self.w_qkv, slabs=True)
+        proj = rt.linear(x, self.w_qkv, slabs=True)
         norm = "none" if s.qk_norm_eps is None else ("weighted" if s.qk_norm_weight else "plain")
         coef, every = s.q_temp if s.q_temp is not None else (0.0, 0)
         # (without projections of its own only q was projected: its columns stand at the row's start all the same)
@@ -238,7 +237,8 @@ class Attention:
                                 s.qk_norm_eps or 0.0, self.q_norm, self.k_norm, coef, every,
                                 write_kv=cache.writable and s.own_kv,
                                 q_head_scale=self.head_temp_capped if capped else self.head_temp, v_norm_eps=s.v_norm_eps,
-                                angles=angles, rotary_dim=rotary_dim, v_first_in=v_in, v_first_out=v_out, v_lambda=self.v_lambda)
+                                angles=angles, rotary_dim=rotary_dim, v_first_in=v_in, v_first_out=v_out, v_lambda=self.v_lambda,
+                                interleaved=getattr(self.position, "pairing", "half") == "interleaved", keys_as_values=s.keys_as_values)
         if rt.dtype == "bfloat16" and not fast:
             rt.generic_attention_launches += 1
         padded = fast and wide_rows             # results as wide as the keys, zeros beyond the value's width
@@ -348,22 +348,23 @@ def decode_workspace(rt, batch, num_heads, head_dim):
 @register("mixer", "parallel_mixer")
 class ParallelMixer:
     """Two mixers side by side on the same input (`ParallelMixerSpec`): delta = left_scale left(x) + right_scale right(x),
-    handed on as a weighted sum of the two results, which the block adds to the residual stream term by term.  One of them
+    handed on as a weighted sum of the two results, which the block adds to the residual stream term by term; where the two
+    results are normed first, as a sum of normed results, which the next norm carries out in its own kernel.  One of them
     may keep keys and values in pages and one a state of fixed size; each gets what it asked for."""
 
     def __init__(self, spec, runtime):
-        from .base import part_class
         self.spec = spec
         self.rt = runtime
         self.sides = [part_class("mixer", side.kind)(side, runtime) for side in (spec.left, spec.right)]
         self.scales = (float(spec.left_scale), float(spec.right_scale))
+        self.norms = [build_part("norm", norm, runtime) for norm in (spec.left_norm, spec.right_norm) if norm is not None]
         self.graph_safe = all(getattr(side, "graph_safe", False) for side in self.sides)
+        self.takes_scaled_rows = all(getattr(side, "takes_scaled_rows", False) for side in self.sides)
         if sum(side.cache_need() is not None for side in self.sides) > 1 or sum(side.state_need() is not None for side in self.sides) > 1:
             raise ValueError("of two mixers side by side at most one keeps keys and values and at most one a state")
 
     @staticmethod
     def _side_classes(spec):
-        from .base import part_class
         return [(side, part_class("mixer", side.kind)) for side in (spec.left, spec.right)]
 
     @classmethod
@@ -371,6 +372,9 @@ class ParallelMixer:
         out = {}
         for side, side_cls in cls._side_classes(spec):
             out.update({side.prefix + name: p for name, p in side_cls.params(side).items()})
+        for norm in (spec.left_norm, spec.right_norm):
+            if norm is not None:
+                out.update(part_params("norm", norm))
         return out
 
     @classmethod
@@ -378,6 +382,9 @@ class ParallelMixer:
         out = {}
         for side, side_cls in cls._side_classes(spec):
             out.update({side.prefix + name: how for name, how in getattr(side_cls, "placement", lambda s: {})(side).items()})
+        for norm in (spec.left_norm, spec.right_norm):
+            if norm is not None:
+                out.update({norm.prefix + name: how for name, how in part_class("norm", norm.kind).placement(norm).items()})
         return out
 
     @classmethod
@@ -401,6 +408,9 @@ class ParallelMixer:
         for side in self.sides:
             prefix = side.spec.prefix
             side.load({name[len(prefix):]: t for name, t in tensors.items() if name.startswith(prefix)})
+        for norm in self.norms:
+            prefix = norm.spec.prefix
+            norm.load({name[len(prefix):]: t for name, t in tensors.items() if name.startswith(prefix)})
 
     def cache_need(self):
         return next((need for need in (side.cache_need() for side in self.sides) if need is not None), None)
@@ -410,9 +420,13 @@ class ParallelMixer:
 
     def forward(self, x, batch, cache, state):
         from ..runtime import WeightedDelta
+        results = [side.forward(x, batch, cache if side.cache_need() is not None else None, state if side.state_need() is not None else None)
+                   for side in self.sides]
+        if self.norms:
+            from .norm import NormedSum
+            return NormedSum(self.rt, [(self.rt.settle(delta), norm, scale) for delta, norm, scale in zip(results, self.norms, self.scales)])
         total = None
-        for side, scale in zip(self.sides, self.scales):
-            delta = side.forward(x, batch, cache if side.cache_need() is not None else None, state if side.state_need() is not None else None)
+        for delta, scale in zip(results, self.scales):
             term = WeightedDelta.of(self.rt, delta, scale)
             total = term if total is None else total.plus(term)
         return total

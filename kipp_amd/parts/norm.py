@@ -60,6 +60,8 @@ class RMSNorm:
             if fused is not None:
                 return fused
             delta = delta.run()
+        elif isinstance(delta, NormedSum):
+            return delta.add_to(x, self, self.rt.empty(x.shape, out_dtype))
         elif isinstance(delta, WeightedDelta):
             delta.add_to(x)         # every term where it lies, then the norm alone
             return self.forward(x, out_dtype)
@@ -119,6 +121,27 @@ class NormedDelta(Pending):
                                          next_norm.weight if next_norm is not None else None,
                                          next_norm.bias if next_norm is not None else None,
                                          next_norm.spec.eps if next_norm is not None else 0.0, out)
+
+
+class NormedSum(Pending):
+    """Results that are each still to be RMS-normed, scaled and added: x += sum_i scale_i N_i(delta_i).  `terms`: one or two of
+    (delta, norm, scale), delta a float32 tensor or its slabs, norm an `RMSNorm`.  An RMS norm that follows carries it out in its
+    own kernel (`add_to` with that norm and a tensor for its rows); `run()` gives the sum as a tensor."""
+    __slots__ = ("rt", "terms")
+
+    def __init__(self, rt, terms):
+        self.rt, self.terms = rt, [tuple(t) for t in terms]
+
+    def add_to(self, x, next_norm=None, out=None):
+        self.rt.ops.normed_sum_step(x, [(delta, norm.weight, norm.spec.eps, scale) for delta, norm, scale in self.terms],
+                                    next_norm.weight if next_norm is not None else None,
+                                    next_norm.spec.eps if next_norm is not None else 0.0, out)
+        return x if out is None else out
+
+    def run(self):
+        import torch
+        shape = tuple(self.terms[0][0].shape[-2:])
+        return self.add_to(self.rt.ops.fill_zero(self.rt.empty(shape, torch.float32)))
 
 
 @register("norm", "layer_norm")

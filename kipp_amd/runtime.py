@@ -369,6 +369,27 @@ class Runtime:
         self.library_products += 1
         return library()
 
+    def squared_relu(self, x, w: "Weight", act: torch.Tensor) -> torch.Tensor:
+        """act [M, N] (bfloat16) = relu(x . w^T)^2 for many rows: our kernel ends in the activation; after the library's
+        product (float32, so that either way rounds once) it is a kernel of its own."""
+        m, k = x.shape
+        rows = w.rows
+
+        def ours(force=0):
+            return self.ops.gemm_tiles(x, rows, end="relu2", force=force)
+
+        def library():
+            return self.ops.activate(self._library_product(x, rows), act, "relu2")
+        if self.ops.gemm_tiles_ok(m, k, rows.shape[0]):
+            ways = {"library": library, "plan": ours}
+            ways.update({cut: (lambda cut=cut: ours(cut)) for cut in self.TILE_CUTS_BF16})
+            choice = self._fastest(("relu2", self._rows_class(m), rows.shape[0], k), ways, ("plan",) + self.TILE_CUTS_BF16)
+            if choice != "library":
+                self.tile_products += 1
+                return ours(0 if choice == "plan" else choice)
+        self.library_products += 1
+        return library()
+
     def linear(self, x, w, slabs: bool = False, defer: bool = False, x_steps_major: bool = False):
         """float32 [M, N] = x [M, K] . w [N, K]^T.  With `slabs` the result may come
         as [parts, M, N] whose sum over parts is the product (few rows against a
