@@ -374,6 +374,41 @@ def bipazen_config(qwen: dict, layers: int, kind: str) -> dict:
     return {"architecture": "Bipazen", "vocab": qwen["vocab_size"], "width": width, "norm": {"eps": 1e-6}, "max_position": 8192, "layers": made}
 
 
+def bavedra_config(qwen: dict, layers: int, kind: str) -> dict:
+    """A Bavedra configuration with the layer sizes of a Qwen3 shape (width, vocabulary, as many feed-forward weights) and
+    `layers` layers of one kind, so that every mechanism's kernels stand beside their like alone: "parallel" (Qwen3's heads and
+    head size with a window of 1,024 keys, half the head turned, beside a state space layer of width / 64 heads of 64 with a state
+    of 128 and a filter of 4 taps: Zivazen's parallel layer; dense), "delta" (8 heads, keys of 128 or 256, values that fill the
+    width, one query/key head for every two heads, 4 taps: Bebulorn's; dense), "rglru" (as wide as the model, in blocks of 256
+    channels, 4 taps: Bipazen's; dense), "moe" (the recurrence with the routed feed-forward: 32 gated experts of a quarter of the
+    dense inner size and 8 identity experts in 8 groups of which 4 stay, 4 choices a token, and a shared expert as large), or
+    "mixed" (parallel + dense, delta + routed, rglru + routed, parallel + routed, a layer beyond the fourth with the weights of
+    the one four before it).  The dense feed-forward has no gate and an inner size half as large again, which is as many weights
+    as the gated one's."""
+    width, heads, ff = qwen["hidden_size"], qwen["num_attention_heads"], qwen["intermediate_size"]
+    head_dim = qwen.get("head_dim") or width // heads
+    left = {"heads": heads, "kv_heads": qwen["num_key_value_heads"], "dim": head_dim, "vdim": head_dim, "scale": head_dim ** -0.5,
+            "mask": {"size": 1024}, "rot": {"base": 10000.0, "dims": head_dim // 2}}
+    right = {"heads": width // 64, "vdim": 64, "state": 128, "groups": 1, "conv": 4, "norm_groups": 1}
+    mixers = {"parallel": {"left": left, "right": right},
+              "delta": {"heads": 8, "kv_heads": 4, "dim": 128 if width <= 2560 else 256, "vdim": width // 8, "conv": 4},
+              "rglru": {"width": width, "blocks": width // 256, "conv": 4}}
+    dense = {"kind": "dense", "ff": ff * 3 // 2}
+    moe = {"kind": "moe", "router": {"experts": 32, "identity": 8, "top": 4, "groups": {"count": 8, "keep": 4}}, "expert": {"ff": ff // 4},
+           "shared": {"ff": ff // 4}}
+    kinds = {"parallel": [("parallel", dense)], "delta": [("delta", dense)], "rglru": [("rglru", dense)], "moe": [("rglru", moe)],
+             "mixed": [("parallel", dense), ("delta", moe), ("rglru", moe), ("parallel", moe)]}
+    order = kinds[kind]
+    made = []
+    for i in range(layers):
+        name, mlp = order[i % len(order)]
+        made.append({"type": name, "mixer": json.loads(json.dumps(mixers[name])), "mlp": json.loads(json.dumps(mlp))})
+        if kind == "mixed" and i >= len(order):
+            made[-1]["weights_of"] = i % len(order)
+    return {"architecture": "Bavedra", "vocab": qwen["vocab_size"], "width": width, "embedding": {"scale": 1.0}, "norm": {"eps": 1e-6},
+            "max_position": 8192, "layers": made}
+
+
 def design_points(config, args, label):
     """Prefill of one 2,048-token prompt and decode steps at two batch sizes behind such prompts, for one model made
     with random weights: milliseconds, tokens a second, and what the kernels ran as (recorded steps, library products,
@@ -506,6 +541,30 @@ def bipazen_bench(args) -> int:
     return 0
 
 
+def bavedra_bench(args) -> int:
+    """`--design bavedra`: the Bavedra design beside Qwen3 and beside the layers that are closest to its own (Zivazen's window
+    attention beside a state space layer, Bebulorn's delta rule and routed feed-forward, Bipazen's recurrence) at equal layer
+    sizes, a few layers of each, random weights: one model for each of its mechanisms alone, and one with all of them in turn."""
+    from kipp_amd.config import shape_config
+    layers = args.layers or 4
+    kinds = args.design_kinds if args.design_kinds != DESIGN_KINDS_DEFAULT else "parallel,delta,rglru,moe,mixed"
+    sizes = {}
+    for shape in [s for s in args.design_shapes.split(",") if s]:
+        qwen = shape_config(shape)
+        qwen["num_hidden_layers"] = layers
+        sizes[shape] = {"qwen3": design_points(qwen, args, f"{shape} qwen3"),
+                        "zivazen_parallel": design_points(zivazen_config(qwen, layers, "parallel"), args, f"{shape} zivazen, parallel"),
+                        "bebulorn_delta": design_points(bebulorn_config(qwen, layers, "delta"), args, f"{shape} bebulorn, delta"),
+                        "bebulorn_moe": design_points(bebulorn_config(qwen, layers, "moe"), args, f"{shape} bebulorn, moe"),
+                        "bipazen_rglru": design_points(bipazen_config(qwen, layers, "rglru"), args, f"{shape} bipazen, rglru")}
+        for kind in [k for k in kinds.split(",") if k]:
+            sizes[shape][f"bavedra_{kind}"] = design_points(bavedra_config(qwen, layers, kind), args, f"{shape} bavedra, {kind}")
+    print(json.dumps({"metric": "prefill and decode of the Bavedra design beside Qwen3 and the closest layers of other designs at equal layer sizes (bf16, random weights)",
+                      "design": "bavedra", "layers": layers, "prompt_tokens": args.prompt, "steps": args.steps,
+                      "unit": "ms and tok/s", "n_gpus": 1, "dtype": "bf16", "data": "synthetic", "sizes": sizes}), flush=True)
+    return 0
+
+
 def design_bench(args) -> int:
     """`--design tobinex`: the Tobinex design beside Qwen3 at equal layer sizes (both with every key kept, and Tobinex
     once more with a window of 1,024 keys behind 4 kept ones), a few layers of each, random weights."""
@@ -545,12 +604,13 @@ def main():
     ap.add_argument("--no-c-host", action="store_true", help="leave out the points measured through the C host")
     ap.add_argument("--products", choices=["default", "own", "auto", "library"], default="default",
                     help="products of many rows (prompt portions): the runtime's default, our kernel only, the fastest of ours and the library's, the library's")
-    ap.add_argument("--design", choices=["tobinex", "rerizen", "bebulorn", "zivazen", "bipazen"], default=None,
+    ap.add_argument("--design", choices=["tobinex", "rerizen", "bebulorn", "zivazen", "bipazen", "bavedra"], default=None,
                     help="instead of the default workload: this design beside Qwen3 at equal layer sizes (prefill and decode, a few layers)")
     ap.add_argument("--design-shapes", default="qwen3-4b,qwen3-8b", help="the Qwen3 shapes whose layer sizes --design takes")
     ap.add_argument("--design-kinds", default=DESIGN_KINDS_DEFAULT,
-                    help="--design rerizen, bebulorn, zivazen or bipazen: the models that are measured, one mechanism each or all in turn "
-                         "(bebulorn: attention,lightning,delta,moe,mixed; zivazen: attention,attention_narrow,parallel,moe,mixed; bipazen: mamba2,rglru,latent,mixed)")
+                    help="--design rerizen, bebulorn, zivazen, bipazen or bavedra: the models that are measured, one mechanism each or all in turn "
+                         "(bebulorn: attention,lightning,delta,moe,mixed; zivazen: attention,attention_narrow,parallel,moe,mixed; bipazen: mamba2,rglru,latent,mixed; "
+                         "bavedra: parallel,delta,rglru,moe,mixed)")
     args = ap.parse_args()
     if args.gpus != 1:
         print(f"bench: this engine runs on one GPU; --gpus {args.gpus} is not supported")
@@ -561,6 +621,8 @@ def main():
         return bebulorn_bench(args)
     if args.design == "bipazen":
         return bipazen_bench(args)
+    if args.design == "bavedra":
+        return bavedra_bench(args)
     if args.design == "zivazen":
         return zivazen_bench(args)
     if args.design:
