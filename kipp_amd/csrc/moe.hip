@@ -51,17 +51,18 @@ __device__ __forceinline__ float activate(float z, int act) {
     }
 }
 
-// One wave a token.  z: float32 [tokens][stride] (or slabs of it, added in order).
+// One wave a token, a lane REGS of the experts.  z: float32 [tokens][stride] (or slabs of it, added in order).
+template <int REGS>
 __global__ void __launch_bounds__(ROUTE_WAVES * KIPP_WAVE)
 moe_route_kernel(const float* __restrict__ z, int parts, size_t part_stride, int stride, int32_t* __restrict__ chosen,
                  float* __restrict__ weight, int tokens, int experts, int top, float eps) {
     const int wave = threadIdx.x / KIPP_WAVE, lane = threadIdx.x & (KIPP_WAVE - 1);
     const int t = blockIdx.x * ROUTE_WAVES + wave;
     if (t >= tokens) return;        // no barrier below
-    float p[MAX_EXPERTS / KIPP_WAVE];
+    float p[REGS];
     float m = -INFINITY;
 #pragma unroll
-    for (int i = 0; i < MAX_EXPERTS / KIPP_WAVE; ++i) {
+    for (int i = 0; i < REGS; ++i) {
         const int e = lane + i * KIPP_WAVE;
         float v = -INFINITY;
         if (e < experts) {
@@ -74,7 +75,7 @@ moe_route_kernel(const float* __restrict__ z, int parts, size_t part_stride, int
     m = wave_max(m);
     float sum = 0.0f;
 #pragma unroll
-    for (int i = 0; i < MAX_EXPERTS / KIPP_WAVE; ++i) {
+    for (int i = 0; i < REGS; ++i) {
         p[i] = (lane + i * KIPP_WAVE < experts) ? expf(p[i] - m) : -1.0f;
         if (p[i] > 0.0f) sum += p[i];
     }
@@ -86,7 +87,7 @@ moe_route_kernel(const float* __restrict__ z, int parts, size_t part_stride, int
         float best = -1.0f;
         int best_e = MAX_EXPERTS;
 #pragma unroll
-        for (int i = 0; i < MAX_EXPERTS / KIPP_WAVE; ++i)
+        for (int i = 0; i < REGS; ++i)
             if (p[i] > best) { best = p[i]; best_e = lane + i * KIPP_WAVE; }     // the lowest index of a lane's largest
         for (int off = 32; off > 0; off >>= 1) {
             const float ob = __shfl_xor(best, off, KIPP_WAVE);
@@ -94,7 +95,7 @@ moe_route_kernel(const float* __restrict__ z, int parts, size_t part_stride, int
             if (ob > best || (ob == best && oe < best_e)) { best = ob; best_e = oe; }
         }
 #pragma unroll
-        for (int i = 0; i < MAX_EXPERTS / KIPP_WAVE; ++i)
+        for (int i = 0; i < REGS; ++i)
             if (lane + i * KIPP_WAVE == best_e) p[i] = -1.0f;
         const float s = best / sum;
         picked_sum += s;
@@ -108,21 +109,22 @@ moe_route_kernel(const float* __restrict__ z, int parts, size_t part_stride, int
 
 // One wave a token: sigmoid scores (`softmax`: a softmax over all of them), a correction for the choice alone, groups of
 // neighbouring experts of which the best stay (by the sum of their two largest, or, `by_largest`, by their largest).
+template <int REGS>
 __global__ void __launch_bounds__(ROUTE_WAVES * KIPP_WAVE)
 moe_route_grouped_kernel(const float* __restrict__ z, int parts, size_t part_stride, int stride, const float* __restrict__ correction,
                          int32_t* __restrict__ chosen, float* __restrict__ weight, int tokens, int experts, int top, float eps,
                          int group_count, int group_keep, float scale, int renormalize, int softmax, int by_largest) {
-    __shared__ float c_s[ROUTE_WAVES][MAX_EXPERTS];     // choice scores, then -inf for experts of groups that do not stay
-    __shared__ float g_s[ROUTE_WAVES][MAX_EXPERTS];     // group scores, -inf once a group is taken
+    __shared__ float c_s[ROUTE_WAVES][REGS * KIPP_WAVE];     // choice scores, then -inf for experts of groups that do not stay
+    __shared__ float g_s[ROUTE_WAVES][REGS * KIPP_WAVE];     // group scores, -inf once a group is taken
     const int wave = threadIdx.x / KIPP_WAVE, lane = threadIdx.x & (KIPP_WAVE - 1);
     int t = blockIdx.x * ROUTE_WAVES + wave;
     const bool live = t < tokens;
     if (!live) t = tokens - 1;      // stay in step with the barriers
     const int size = experts / group_count;
-    float s[MAX_EXPERTS / KIPP_WAVE];
+    float s[REGS];
     float m = -INFINITY;
 #pragma unroll
-    for (int i = 0; i < MAX_EXPERTS / KIPP_WAVE; ++i) {
+    for (int i = 0; i < REGS; ++i) {
         const int e = lane + i * KIPP_WAVE;
         s[i] = 0.0f;
         if (e < experts) {
@@ -136,17 +138,17 @@ moe_route_grouped_kernel(const float* __restrict__ z, int parts, size_t part_str
         m = wave_max(m);
         float sum = 0.0f;
 #pragma unroll
-        for (int i = 0; i < MAX_EXPERTS / KIPP_WAVE; ++i)
+        for (int i = 0; i < REGS; ++i)
             if (lane + i * KIPP_WAVE < experts) {
                 s[i] = expf(s[i] - m);
                 sum += s[i];
             }
         sum = wave_sum(sum);
 #pragma unroll
-        for (int i = 0; i < MAX_EXPERTS / KIPP_WAVE; ++i) s[i] = s[i] / sum;
+        for (int i = 0; i < REGS; ++i) s[i] = s[i] / sum;
     }
 #pragma unroll
-    for (int i = 0; i < MAX_EXPERTS / KIPP_WAVE; ++i) {
+    for (int i = 0; i < REGS; ++i) {
         const int e = lane + i * KIPP_WAVE;
         if (e < experts) c_s[wave][e] = s[i] + (correction != nullptr ? correction[e] : 0.0f);
     }
@@ -161,29 +163,42 @@ moe_route_grouped_kernel(const float* __restrict__ z, int parts, size_t part_str
             g_s[wave][g] = size > 1 && !by_largest ? a + b : a;
         }
         __syncthreads();
-        for (int round = 0; round < group_keep; ++round) {
-            float best = -INFINITY;
-            int best_g = MAX_EXPERTS;
-            for (int g = lane; g < group_count; g += KIPP_WAVE) {
+        if (group_count <= KIPP_WAVE) {
+            // a lane a group: it stays if fewer than `keep` groups come before it (a larger score, or as large with a lower index)
+            const float mine_g = lane < group_count ? g_s[wave][lane] : 0.0f;
+            int before = 0;
+            for (int g = 0; g < group_count; ++g) {
                 const float v = g_s[wave][g];
-                if (v > best || (best_g == MAX_EXPERTS && v != -INFINITY)) { best = v; best_g = g; }
-            }
-            for (int off = 32; off > 0; off >>= 1) {
-                const float ob = __shfl_xor(best, off, KIPP_WAVE);
-                const int og = __shfl_xor(best_g, off, KIPP_WAVE);
-                if (og != MAX_EXPERTS && (best_g == MAX_EXPERTS || ob > best || (ob == best && og < best_g))) { best = ob; best_g = og; }
+                before += v > mine_g || (v == mine_g && g < lane) ? 1 : 0;
             }
             __syncthreads();
-            if (lane == 0 && best_g != MAX_EXPERTS) g_s[wave][best_g] = -INFINITY;      // taken: it stays
+            if (lane < group_count && before < group_keep) g_s[wave][lane] = -INFINITY;         // taken: it stays
             __syncthreads();
+        } else {
+            for (int round = 0; round < group_keep; ++round) {
+                float best = -INFINITY;
+                int best_g = MAX_EXPERTS;
+                for (int g = lane; g < group_count; g += KIPP_WAVE) {
+                    const float v = g_s[wave][g];
+                    if (v > best || (best_g == MAX_EXPERTS && v != -INFINITY)) { best = v; best_g = g; }
+                }
+                for (int off = 32; off > 0; off >>= 1) {
+                    const float ob = __shfl_xor(best, off, KIPP_WAVE);
+                    const int og = __shfl_xor(best_g, off, KIPP_WAVE);
+                    if (og != MAX_EXPERTS && (best_g == MAX_EXPERTS || ob > best || (ob == best && og < best_g))) { best = ob; best_g = og; }
+                }
+                __syncthreads();
+                if (lane == 0 && best_g != MAX_EXPERTS) g_s[wave][best_g] = -INFINITY;      // taken: it stays
+                __syncthreads();
+            }
         }
         for (int e = lane; e < experts; e += KIPP_WAVE)
             if (g_s[wave][e / size] != -INFINITY) c_s[wave][e] = -INFINITY;             // its group was not taken
         __syncthreads();
     }
-    float c[MAX_EXPERTS / KIPP_WAVE];
+    float c[REGS];
 #pragma unroll
-    for (int i = 0; i < MAX_EXPERTS / KIPP_WAVE; ++i) {
+    for (int i = 0; i < REGS; ++i) {
         const int e = lane + i * KIPP_WAVE;
         c[i] = e < experts ? c_s[wave][e] : -INFINITY;
     }
@@ -193,7 +208,7 @@ moe_route_grouped_kernel(const float* __restrict__ z, int parts, size_t part_str
         float best = -INFINITY, best_s = 0.0f;
         int best_e = MAX_EXPERTS;
 #pragma unroll
-        for (int i = 0; i < MAX_EXPERTS / KIPP_WAVE; ++i)
+        for (int i = 0; i < REGS; ++i)
             if (c[i] > best) { best = c[i]; best_e = lane + i * KIPP_WAVE; best_s = s[i]; }     // the lowest index of a lane's largest
         for (int off = 32; off > 0; off >>= 1) {
             const float ob = __shfl_xor(best, off, KIPP_WAVE), os = __shfl_xor(best_s, off, KIPP_WAVE);
@@ -201,7 +216,7 @@ moe_route_grouped_kernel(const float* __restrict__ z, int parts, size_t part_str
             if (ob > best || (ob == best && oe < best_e)) { best = ob; best_e = oe; best_s = os; }
         }
 #pragma unroll
-        for (int i = 0; i < MAX_EXPERTS / KIPP_WAVE; ++i)
+        for (int i = 0; i < REGS; ++i)
             if (lane + i * KIPP_WAVE == best_e) c[i] = -INFINITY;
         picked_sum += best_s;
         if (lane == j) { mine = best_s; mine_e = best_e < experts ? best_e : 0; }
@@ -563,8 +578,13 @@ extern "C" int kipp_moe_route(const float* z, int parts, int stride, int32_t* ch
     const int pairs = tokens * top;
     if (tile_rows != TILE_ROWS && tile_rows != MFMA_ROWS) return -1;
     if (max_tiles < (pairs + tile_rows - 1) / tile_rows + (experts < pairs ? experts : pairs)) return -1;
-    hipLaunchKernelGGL(moe_route_kernel, dim3((tokens + ROUTE_WAVES - 1) / ROUTE_WAVES), dim3(ROUTE_WAVES * KIPP_WAVE), 0, stream, z, parts,
-                       (size_t)tokens * stride, stride, chosen, weight, tokens, experts, top, eps);
+#define KIPP_RT(REGS)                                                                                                                  \
+    hipLaunchKernelGGL(moe_route_kernel<REGS>, dim3((tokens + ROUTE_WAVES - 1) / ROUTE_WAVES), dim3(ROUTE_WAVES * KIPP_WAVE), 0, stream, z, \
+                       parts, (size_t)tokens * stride, stride, chosen, weight, tokens, experts, top, eps)
+    if (experts <= KIPP_WAVE) KIPP_RT(1);
+    else if (experts <= 4 * KIPP_WAVE) KIPP_RT(4);
+    else KIPP_RT(MAX_EXPERTS / KIPP_WAVE);
+#undef KIPP_RT
     hipLaunchKernelGGL(moe_sort_kernel, dim3(1), dim3(1024), 0, stream, (const int32_t*)chosen, pairs, experts, top, pair_token,
                        place_of_pair, tiles, max_tiles, tile_rows, (const float*)weight, row_weight);
     return KIPP_LAUNCH_CHECK();
@@ -585,9 +605,14 @@ extern "C" int kipp_moe_route_grouped(const float* z, int parts, int stride, con
     const int pairs = tokens * top, real = experts - identity;
     if (tile_rows != TILE_ROWS && tile_rows != MFMA_ROWS) return -1;
     if (max_tiles < (pairs + tile_rows - 1) / tile_rows + (real < pairs ? real : pairs)) return -1;
-    hipLaunchKernelGGL(moe_route_grouped_kernel, dim3((tokens + ROUTE_WAVES - 1) / ROUTE_WAVES), dim3(ROUTE_WAVES * KIPP_WAVE), 0, stream, z,
-                       parts, (size_t)tokens * stride, stride, correction, chosen, weight, tokens, experts, top, eps, group_count, group_keep,
-                       scale, renormalize, softmax, by_largest);
+#define KIPP_RG(REGS)                                                                                                                     \
+    hipLaunchKernelGGL(moe_route_grouped_kernel<REGS>, dim3((tokens + ROUTE_WAVES - 1) / ROUTE_WAVES), dim3(ROUTE_WAVES * KIPP_WAVE), 0, stream, \
+                       z, parts, (size_t)tokens * stride, stride, correction, chosen, weight, tokens, experts, top, eps, group_count, group_keep, \
+                       scale, renormalize, softmax, by_largest)
+    if (experts <= KIPP_WAVE) KIPP_RG(1);
+    else if (experts <= 4 * KIPP_WAVE) KIPP_RG(4);
+    else KIPP_RG(MAX_EXPERTS / KIPP_WAVE);
+#undef KIPP_RG
     hipLaunchKernelGGL(moe_sort_kernel, dim3(1), dim3(1024), 0, stream, (const int32_t*)chosen, pairs, real, top, pair_token,
                        place_of_pair, tiles, max_tiles, tile_rows, (const float*)weight, row_weight);
     return KIPP_LAUNCH_CHECK();
